@@ -1,3 +1,5 @@
+from .bilolix import (BilolixConfig, BilolixLayer, ChannelDeltaConfig, FadingConfig, GeluFFConfig, MapAttentionConfig, PairTurn,
+                      SoftmaxMoEConfig)
 from .fazezen import (ChunkedAttentionConfig, DenseConfig, FazezenConfig, FazezenLayer, LightningConfig, ParallelConfig,
                       RetentionConfig, Rotation, Stretch)
 from .kuditar import (ChannelDecayConfig, DeltaRuleConfig, DenseFFConfig, GatedAttentionConfig, KuditarConfig, KuditarLayer,
@@ -8,7 +10,7 @@ from .registry import (architecture_of, load_config, register_architecture, regi
                        unregister_architecture)
 from .togalorn import ExpertConfig, LatentMixerConfig, LoopConfig, Mamba2MixerConfig, MoEConfig, TogalornConfig, TogalornLayer
 from .spec import (AttentionSpec, BlockSpec, ClampedGLUSpec, GatedDeltaSpec, GatedLinearSpec, GatedMLPSpec, GroupRMSNormSpec,
-                   LatentAttentionSpec, LayerCall, LayerNormSpec, LinearAttentionSpec, MixerPairSpec,
+                   LatentAttentionSpec, LayerCall, LayerNormSpec, LinearAttentionSpec, MapAttentionSpec, MixerPairSpec, MLPSpec,
                    ModelSpec, NoPositionSpec, OutNormBlockSpec, ParallelBlockSpec, RMSNormSpec, ReentrySpec, RopeSpec,
                    RoutedMoESpec, ScaledRopeSpec, SharedNormBlockSpec, ShortConvSpec, StateSpaceSpec, StretchedRopeSpec,
                    SwiGLUSpec, TableMoESpec)

@@ -172,6 +172,30 @@ class LatentAttentionSpec:
 
 
 @dataclass(frozen=True)
+class MapAttentionSpec:
+    """Attention as the difference of two softmax maps over one value row.  A head has two queries of ``map_dim`` features
+    (``W_q`` has ``n_heads * 2 * map_dim`` rows, head by head as [map 1, map 2]), its key head two keys laid out the same
+    way and one value of ``value_dim``; ``position`` turns each map's query and key.  With ``o1``, ``o2`` the two maps'
+    softmax-weighted sums (scores ``q . k * scale``, the last ``window`` positions) and
+    ``lam = exp(q1 . k1) - exp(q2 . k2) + share`` (four stored vectors of ``map_dim``: one number for the layer), the head's
+    output is ``(o1 - lam o2) / sqrt(mean((o1 - lam o2)^2) + eps) * (1 - share)``; with ``head_gate`` times
+    ``sigmoid(W_g x)_h``, one number a head."""
+
+    hidden: int
+    n_heads: int
+    n_kv_heads: int
+    map_dim: int
+    value_dim: int
+    position: Any                      # a position-encoding spec (its ``head_dim`` is ``map_dim``)
+    scale: float
+    share: float
+    eps: float
+    window: Optional[int] = None       # keys a query sees, itself included; None = all
+    head_gate: bool = True
+    kind: str = "map_attention"
+
+
+@dataclass(frozen=True)
 class LinearAttentionSpec:
     """Attention without a softmax, through a matrix state per head that fades by a fixed factor a token:
     ``S_t = decay_h S_(t-1) + k_t v_t^T`` (``key_dim x value_dim``, float32, zero at a request's start),
@@ -204,7 +228,12 @@ class GatedDeltaSpec:
     q and k become unit vectors per head (``x / sqrt(sum(x^2) + unit_eps)``), q also times ``key_dim^-0.5``; head ``h``
     uses q/k head ``h // (n_heads / qk_heads)``.  ``beta = sigmoid(W_b x)`` and
     ``g = exp(-exp(A_log) softplus(W_a x + dt_bias))`` per head; ``S <- g S; u = beta (v - S^T k); S <- S + k u^T;
-    o = S^T q``; each head's ``o`` is RMS-normed with a weight of ``value_dim``, times ``silu(W_g x)``, then projected."""
+    o = S^T q``; each head's ``o`` is RMS-normed with a weight of ``value_dim``, times ``silu(W_g x)``, then projected.
+
+    ``decay_rank``: the decay is one a head and key channel, ``g = exp(-exp(A_log_h) softplus(W_up (W_down x) + dt_bias))``
+    with that many features between the two products, and acts on the state's rows (None: one a head, from ``W_a``).
+    ``gate_rank``: the gate's product goes through that many features, ``W_up (W_down x)`` (None: ``W_g x``).
+    ``gate``: the function of it (``"silu"`` or ``"sigmoid"``)."""
 
     hidden: int
     n_heads: int
@@ -215,6 +244,9 @@ class GatedDeltaSpec:
     eps: float
     unit_eps: float = 1e-6
     kind: str = "gated_delta"
+    decay_rank: Optional[int] = None
+    gate_rank: Optional[int] = None
+    gate: str = "silu"
 
 
 @dataclass(frozen=True)
@@ -262,6 +294,17 @@ class SwiGLUSpec:
     hidden: int
     intermediate: int
     kind: str = "swiglu"
+
+
+@dataclass(frozen=True)
+class MLPSpec:
+    """``W_down act(W_up x)``, no gate and no biases; ``activation``: ``"gelu"`` (the error-function form), ``"gelu_tanh"`` or
+    ``"silu"``."""
+
+    hidden: int
+    intermediate: int
+    activation: str = "gelu"
+    kind: str = "mlp"
 
 
 @dataclass(frozen=True)
@@ -334,13 +377,15 @@ class RoutedMoESpec:
     An expert is ``W_down (g sigmoid(alpha g) (u + 1))`` with ``g = min(W_gate x, limit)``,
     ``u = clamp(W_up x, -limit, limit)``.  ``shared_ff``: a further expert of that width and ``shared_limit`` runs for every
     token and is added (None: none).  ``score = "sigmoid"``: the scores are each output's sigmoid instead of their
-    softmax; ``renormalize = False``: the weights are the chosen scores as they are; ``route_scale`` multiplies them."""
+    softmax; ``renormalize = False``: the weights are the chosen scores as they are; ``route_scale`` multiplies them.
+    ``router_bias``: a stored vector is added to the logits.  ``shift``: an expert multiplies by ``u + shift``;
+    ``limit = None``: nothing is clamped (with ``alpha`` 1 and ``shift`` 0 an expert is ``W_down (silu(W_gate x) * W_up x)``)."""
 
     hidden: int
     n_experts: int
     top: int
     expert_ff: int
-    limit: float
+    limit: Optional[float]
     n_identity: int = 0
     alpha: float = 1.702
     correction: bool = True
@@ -350,6 +395,8 @@ class RoutedMoESpec:
     score: str = "softmax"
     renormalize: bool = True
     route_scale: float = 1.0
+    router_bias: bool = False
+    shift: float = 1.0
 
 
 @dataclass(frozen=True)
@@ -416,9 +463,11 @@ class SharedNormBlockSpec:
 class ReentrySpec:
     """Before the schedule entries ``at`` (in their order, ``t = 0, 1, ...``) the stream is mixed with the embedding
     output ``x0`` again: ``x <- W [x; x0] + step[t]`` with ``W (hidden, 2 hidden)`` (the stream's columns first) and
-    ``step (len(at), hidden)``.  The model's names ``reentry.weight`` and ``reentry.step`` say where they are stored."""
+    ``step (len(at), hidden)``.  The model's names ``reentry.weight`` and ``reentry.step`` say where they are stored.
+    ``mix = False``: there is no product, ``x <- x + step[t]``."""
 
     at: Tuple[int, ...]
+    mix: bool = True
 
 
 @dataclass(frozen=True)

@@ -19,7 +19,7 @@ void gs_set_error(const char* fmt, ...) {
 
 extern "C" const char* gs_last_error() { return g_err; }
 
-extern "C" int gs_abi_version() { return 12; }
+extern "C" int gs_abi_version() { return 13; }
 
 // ------------------------------------------------------------------ embedding
 
@@ -739,6 +739,7 @@ extern "C" int gs_add_rmsnorm_pair(float* res, const void* d1, const void* d2, i
 // act 0: silu, z / (1 + exp(-z)); act 1: the tanh form of gelu, 0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))).
 __device__ __forceinline__ float gated_act(float z, int act) {
   if (act == 0) return z / (1.0f + expf(-z));
+  if (act == 2) return 0.5f * z * (1.0f + erff(z * 0.7071067811865476f));
   const float u = 0.7978845608028654f * (z + 0.044715f * z * z * z);
   return 0.5f * z * (1.0f + tanhf(u));
 }
@@ -788,7 +789,7 @@ __global__ void gated_act8_kernel(const TI* __restrict__ in, const float* __rest
 extern "C" int gs_gated_act(const void* in, int in_dtype, const float* bias, void* out, int out_dtype, int T, int F,
                             int act, hipStream_t stream) {
   GS_REQUIRE(T >= 0 && F > 0, "gated_act: bad sizes T=%d F=%d", T, F);
-  GS_REQUIRE(act == 0 || act == 1, "gated_act: unknown activation %d", act);
+  GS_REQUIRE(act >= 0 && act <= 2, "gated_act: unknown activation %d", act);
   const long n = (long)T * F;
   if (n == 0) return 0;
   const bool v8 = F % 8 == 0 && ((uintptr_t)in & 15) == 0 && ((uintptr_t)out & 15) == 0 && ((uintptr_t)bias & 15) == 0;
@@ -808,6 +809,49 @@ extern "C" int gs_gated_act(const void* in, int in_dtype, const float* bias, voi
     GS_REQUIRE(false, "gated_act: unknown dtypes %d %d", in_dtype, out_dtype);
 #undef GS_RUN
   GS_LAUNCH_CHECK("gated_act");
+  return 0;
+}
+
+// ------------------------------------------------------------------ an activation alone
+
+// out[i] = act(in[i]): act 0 silu, 1 gelu (tanh form), 2 gelu (error-function form); float32 arithmetic.  VEC: eight values
+// a thread with 16-byte accesses.
+template <typename TI, typename TO, bool VEC>
+__global__ void activate_kernel(const TI* __restrict__ in, TO* __restrict__ out, long n, int act) {
+  const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i >= n) return;
+  if constexpr (VEC) {
+    float v[8];
+    load8f(in + i * 8, v);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) v[e] = gated_act(v[e], act);
+    store8f(out + i * 8, v);
+  } else {
+    out[i] = from_f32<TO>(gated_act(to_f32(in[i]), act));
+  }
+}
+
+extern "C" int gs_activate(const void* in, int in_dtype, void* out, int out_dtype, long n, int act, hipStream_t stream) {
+  GS_REQUIRE(n >= 0, "activate: bad size");
+  GS_REQUIRE(act >= 0 && act <= 2, "activate: unknown activation %d", act);
+  if (n == 0) return 0;
+  const bool v8 = n % 8 == 0 && ((uintptr_t)in & 15) == 0 && ((uintptr_t)out & 15) == 0;
+  const int blocks = gs_ceil_div(v8 ? n / 8 : n, 256);
+#define GS_RUN(TI, TO)                                                                                        \
+  do {                                                                                                        \
+    if (v8) activate_kernel<TI, TO, true><<<blocks, 256, 0, stream>>>((const TI*)in, (TO*)out, n / 8, act);    \
+    else activate_kernel<TI, TO, false><<<blocks, 256, 0, stream>>>((const TI*)in, (TO*)out, n, act);          \
+  } while (0)
+  if (in_dtype == GS_F32 && out_dtype == GS_F32)
+    GS_RUN(float, float);
+  else if (in_dtype == GS_F32 && out_dtype == GS_BF16)
+    GS_RUN(float, bf16);
+  else if (in_dtype == GS_BF16 && out_dtype == GS_BF16)
+    GS_RUN(bf16, bf16);
+  else
+    GS_REQUIRE(false, "activate: unknown dtypes %d %d", in_dtype, out_dtype);
+#undef GS_RUN
+  GS_LAUNCH_CHECK("activate");
   return 0;
 }
 

@@ -29,6 +29,8 @@
 // delta_rule_prep: what the gated delta rule computes between its convolutions and the recurrence, in float32:
 //   q <- q / sqrt(sum q^2 + unit_eps) * q_scale,  k <- k / sqrt(sum k^2 + unit_eps)        per (token, q/k head), in place
 //   g = exp(-exp(A_log[h]) softplus(a + dt_bias[h])),  beta = sigmoid(b)                     per (token, head)
+//   with `channels` the decay is one a key channel: on float32 products z (T, ldz), in place in the columns [oz, oz + H n),
+//   z[h n + i] <- exp(-exp(A_log[h]) softplus(z[h n + i] + dt_bias[h n + i])); the gates are then beta alone (T, H)
 // channel_decay: alpha = sigmoid(z)^(1/tau) = exp(-softplus(-z) / tau), elementwise in place.
 #include "common.h"
 
@@ -354,7 +356,8 @@ extern "C" int gs_gated_state_chain(const float* M, const float* B, float* first
   return 0;
 }
 
-// One block of 256 threads per token: a wavefront per q or k head in turn, then the heads' gates.
+// One block of 256 threads per token: a wavefront per q or k head in turn, then the heads' gates (and, with `channels`, the
+// channels' decays).
 //   c (T, ldc) float32: q heads at [0, G n), k heads at [G n, 2 G n), normed in place
 //   rows (T, ldr): the decay's product at [oa + h], the write strength's at [obeta + h]
 //   gates (T, 2 H) float32: g at [h], beta at [H + h]
@@ -362,7 +365,8 @@ template <typename TR>
 __global__ void __launch_bounds__(256)
 delta_rule_prep_kernel(float* __restrict__ c, int ldc, int G, int n, float q_scale, float unit_eps,
                        const TR* __restrict__ rows, int ldr, int oa, int obeta, const float* __restrict__ a_log,
-                       const float* __restrict__ dt_bias, float* __restrict__ gates, int H) {
+                       const float* __restrict__ dt_bias, float* __restrict__ gates, int H, float* __restrict__ z, int ldz,
+                       int oz, int nz) {
   const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   for (int u = wave; u < 2 * G; u += 4) {
     float* v = c + (size_t)t * ldc + (size_t)u * n;
@@ -371,6 +375,14 @@ delta_rule_prep_kernel(float* __restrict__ c, int ldc, int G, int n, float q_sca
     ss = wave_sum(ss);
     const float inv = (u < G ? q_scale : 1.f) / sqrtf(ss + unit_eps);
     for (int i = lane; i < n; i += 64) v[i] *= inv;
+  }
+  if (z) {
+    // (nz: key channels a head)
+    float* zt = z + (size_t)t * ldz + oz;
+    for (int i = threadIdx.x; i < H * nz; i += 256) zt[i] = expf(-expf(a_log[i / nz]) * gr_softplus(zt[i] + dt_bias[i]));
+    for (int h = threadIdx.x; h < H; h += 256)
+      gates[(size_t)t * H + h] = 1.f / (1.f + expf(-to_f32(rows[(size_t)t * ldr + obeta + h])));
+    return;
   }
   for (int h = threadIdx.x; h < H; h += 256) {
     const float a = to_f32(rows[(size_t)t * ldr + oa + h]), b = to_f32(rows[(size_t)t * ldr + obeta + h]);
@@ -381,18 +393,19 @@ delta_rule_prep_kernel(float* __restrict__ c, int ldc, int G, int n, float q_sca
 
 extern "C" int gs_delta_rule_prep(float* c, int ldc, int G, int n, float q_scale, float unit_eps, const void* rows,
                                   int rows_dtype, int ldr, int oa, int obeta, const float* a_log, const float* dt_bias,
-                                  float* gates, int T, int H, hipStream_t stream) {
+                                  float* gates, int T, int H, float* z, int ldz, int oz, hipStream_t stream) {
+  GS_REQUIRE(!z || (oz >= 0 && oz + H * n <= ldz), "delta_rule_prep: the channels' decays lie outside the rows of %d", ldz);
   GS_REQUIRE(T >= 0 && G > 0 && n > 0 && H > 0 && 2 * G * n <= ldc, "delta_rule_prep: bad sizes T=%d G=%d n=%d H=%d ldc=%d",
              T, G, n, H, ldc);
-  GS_REQUIRE(oa >= 0 && obeta >= 0 && oa + H <= ldr && obeta + H <= ldr, "delta_rule_prep: the gates' products lie outside the rows of %d", ldr);
+  GS_REQUIRE((z || (oa >= 0 && oa + H <= ldr)) && obeta >= 0 && obeta + H <= ldr, "delta_rule_prep: the gates' products lie outside the rows of %d", ldr);
   GS_REQUIRE(unit_eps >= 0.f, "delta_rule_prep: bad eps");
   if (T == 0) return 0;
   if (rows_dtype == GS_F32)
     delta_rule_prep_kernel<float><<<T, 256, 0, stream>>>(c, ldc, G, n, q_scale, unit_eps, (const float*)rows, ldr, oa,
-                                                          obeta, a_log, dt_bias, gates, H);
+                                                          obeta, a_log, dt_bias, gates, H, z, ldz, oz, n);
   else if (rows_dtype == GS_BF16)
     delta_rule_prep_kernel<bf16><<<T, 256, 0, stream>>>(c, ldc, G, n, q_scale, unit_eps, (const bf16*)rows, ldr, oa,
-                                                         obeta, a_log, dt_bias, gates, H);
+                                                         obeta, a_log, dt_bias, gates, H, z, ldz, oz, n);
   else
     GS_REQUIRE(false, "delta_rule_prep: unknown dtype %d", rows_dtype);
   GS_LAUNCH_CHECK("delta_rule_prep");

@@ -216,11 +216,14 @@ extern "C" int gs_gated_outnorm(const float* o, const void* gate, int gate_dtype
   GS_REQUIRE(T >= 0 && H > 0 && m > 0, "gated_outnorm: bad sizes T=%d H=%d m=%d", T, H, m);
   GS_REQUIRE(eps > 0.f, "gated_outnorm: eps must be positive");
   GS_REQUIRE(og >= 0 && og + H * m <= ldg, "gated_outnorm: the gate lies outside the rows of %d", ldg);
-  GS_REQUIRE(gate_dtype == out_dtype, "gated_outnorm: gate and result are of one type");
+  GS_REQUIRE(gate_dtype == out_dtype || gate_dtype == GS_F32, "gated_outnorm: the gate is float32 or of the result's type");
   if (T == 0) return 0;
   if (out_dtype == GS_F32)
     gated_outnorm_kernel<float, float><<<T, 256, 0, stream>>>(o, (const float*)gate, ldg, og, w, eps, joint, gate_act,
                                                                (float*)out, H, m);
+  else if (out_dtype == GS_BF16 && gate_dtype == GS_F32)
+    gated_outnorm_kernel<float, bf16><<<T, 256, 0, stream>>>(o, (const float*)gate, ldg, og, w, eps, joint, gate_act,
+                                                              (bf16*)out, H, m);
   else if (out_dtype == GS_BF16)
     gated_outnorm_kernel<bf16, bf16><<<T, 256, 0, stream>>>(o, (const bf16*)gate, ldg, og, w, eps, joint, gate_act,
                                                              (bf16*)out, H, m);

@@ -1,10 +1,11 @@
 // A mixture of gated feed-forwards chosen by a router over the token's own features.
 //
-//   z = W_r x (float32), s = softmax(z) over all router outputs (or, with score_fn 1, s = sigmoid(z), each output for
+//   z = W_r x (+ bias) (float32), s = softmax(z) over all router outputs (or, with score_fn 1, s = sigmoid(z), each output for
 //   itself); the `top` outputs with the largest s + correction are chosen; the chosen ones' weights are their s divided
 //   by the sum of the chosen s (+ 1e-20), or, without `renorm`, their s as they are; both times route_scale.  Outputs e >= E name no
 //   expert with weights: such an "identity expert" gives back its input.  An expert is
-//     g = min(W_gate x, limit), u = clamp(W_up x, -limit, limit), y = W_down (g sigmoid(alpha g) (u + 1)).
+//     g = min(W_gate x, limit), u = clamp(W_up x, -limit, limit), y = W_down (g sigmoid(alpha g) (u + shift))
+//   (limit may be infinite: nothing is clamped).
 //   Expert weights lie stacked: gate_up (E, 2F, H) (a gate's rows, then the up rows), down (E, H, F).
 //
 //   moe_router         one block per token, a wavefront for every four router rows: logits by wavefronts that walk
@@ -18,10 +19,10 @@
 // expert (moe_route with a table of choices) and read every expert's weights once.
 #include "common.h"
 
-__device__ __forceinline__ float clamped_glu(float g, float u, float limit, float alpha) {
+__device__ __forceinline__ float clamped_glu(float g, float u, float limit, float alpha, float shift) {
   g = fminf(g, limit);
   u = fminf(fmaxf(u, -limit), limit);
-  return g / (1.f + expf(-alpha * g)) * (u + 1.f);
+  return g / (1.f + expf(-alpha * g)) * (u + shift);
 }
 
 // A row of H values into LDS as float32, by the whole block: 16-byte reads where the row allows them.
@@ -103,7 +104,8 @@ template <typename T, typename TW>
 __global__ __launch_bounds__(1024) void moe_router_kernel(const T* __restrict__ x, int ldx, const TW* __restrict__ wr,
                                                          const float* __restrict__ correction, int top, int EA, int H,
                                                          int* __restrict__ choice, float* __restrict__ weight,
-                                                         int score_fn, int renorm, float route_scale) {
+                                                         int score_fn, int renorm, float route_scale,
+                                                         const float* __restrict__ bias) {
   extern __shared__ float mr_sh[];           // H floats of the row, EA logits, EA choice scores, top chosen outputs
   float* xs = mr_sh;
   float* z = mr_sh + H;
@@ -150,7 +152,7 @@ __global__ __launch_bounds__(1024) void moe_router_kernel(const T* __restrict__ 
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const float all = wave_sum(s[r]);
-      if (lane == 0 && e0 + r < EA) z[e0 + r] = all;
+      if (lane == 0 && e0 + r < EA) z[e0 + r] = bias ? all + bias[e0 + r] : all;
     }
   }
   __syncthreads();
@@ -160,18 +162,18 @@ __global__ __launch_bounds__(1024) void moe_router_kernel(const T* __restrict__ 
 
 template <typename TI, typename TO>
 __global__ void clamped_glu_kernel(const TI* __restrict__ in, TO* __restrict__ out, int F, long total, float limit,
-                                   float alpha) {
+                                   float alpha, float shift) {
   const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= total) return;
   const long r = i / F;
   const int f = (int)(i % F);
-  out[i] = from_f32<TO>(clamped_glu(to_f32(in[r * 2 * F + f]), to_f32(in[r * 2 * F + F + f]), limit, alpha));
+  out[i] = from_f32<TO>(clamped_glu(to_f32(in[r * 2 * F + f]), to_f32(in[r * 2 * F + F + f]), limit, alpha, shift));
 }
 
 template <typename T, typename TW>
 __global__ void moe_routed_up_kernel(const T* __restrict__ x, int ldx, const int* __restrict__ choice, int top, int E,
                                      const TW* __restrict__ gate_up, int F, int H, float limit, float alpha,
-                                     T* __restrict__ a) {
+                                     float shift, T* __restrict__ a) {
   extern __shared__ float xs[];      // H floats
   const int t = blockIdx.x / top, k = blockIdx.x % top;
   const int e = choice[(size_t)t * top + k];
@@ -206,7 +208,7 @@ __global__ void moe_routed_up_kernel(const T* __restrict__ x, int ldx, const int
     sg = wave_sum(sg);
     su = wave_sum(su);
     // the products are stored in the activation type before the activation, as products of their own would be
-    if (lane == 0) dst[f] = from_f32<T>(clamped_glu(to_f32(from_f32<T>(sg)), to_f32(from_f32<T>(su)), limit, alpha));
+    if (lane == 0) dst[f] = from_f32<T>(clamped_glu(to_f32(from_f32<T>(sg)), to_f32(from_f32<T>(su)), limit, alpha, shift));
   }
 }
 
@@ -302,7 +304,7 @@ static int moe_routed_blocks_y(int outputs, int tokens) {
 
 extern "C" int gs_moe_router(const void* x, int dtype, int ldx, const void* wr, int w_dtype, const float* correction,
                              int top, int EA, int H, int* choice, float* weight, int ntok, int score_fn, int renorm,
-                             float route_scale, hipStream_t stream) {
+                             float route_scale, const float* bias, hipStream_t stream) {
   GS_REQUIRE(score_fn == 0 || score_fn == 1, "moe_router: scores are a softmax (0) or sigmoids (1), not %d", score_fn);
   GS_REQUIRE(ntok >= 0 && top > 0 && EA >= top && H > 0 && ldx >= H, "moe_router: bad sizes T=%d top=%d outputs=%d H=%d", ntok, top, EA, H);
   const size_t lds = ((size_t)H + 2 * (size_t)EA + (size_t)top) * sizeof(float);
@@ -312,13 +314,13 @@ extern "C" int gs_moe_router(const void* x, int dtype, int ldx, const void* wr, 
   const int threads = 64 * (gs_ceil_div(EA, 4) < 16 ? (gs_ceil_div(EA, 4) < 4 ? 4 : gs_ceil_div(EA, 4)) : 16);
   if (dtype == GS_F32 && w_dtype == GS_F32)
     moe_router_kernel<float, float><<<ntok, threads, lds, stream>>>((const float*)x, ldx, (const float*)wr, correction, top,
-                                                                EA, H, choice, weight, score_fn, renorm, route_scale);
+                                                                EA, H, choice, weight, score_fn, renorm, route_scale, bias);
   else if (dtype == GS_BF16 && w_dtype == GS_BF16)
     moe_router_kernel<bf16, bf16><<<ntok, threads, lds, stream>>>((const bf16*)x, ldx, (const bf16*)wr, correction, top, EA, H,
-                                                              choice, weight, score_fn, renorm, route_scale);
+                                                              choice, weight, score_fn, renorm, route_scale, bias);
   else if (dtype == GS_BF16 && w_dtype == GS_F32)
     moe_router_kernel<bf16, float><<<ntok, threads, lds, stream>>>((const bf16*)x, ldx, (const float*)wr, correction, top, EA,
-                                                               H, choice, weight, score_fn, renorm, route_scale);
+                                                               H, choice, weight, score_fn, renorm, route_scale, bias);
   else
     GS_REQUIRE(false, "moe_router: unsupported types %d %d", dtype, w_dtype);
   GS_LAUNCH_CHECK("moe_router");
@@ -326,17 +328,17 @@ extern "C" int gs_moe_router(const void* x, int dtype, int ldx, const void* wr, 
 }
 
 extern "C" int gs_clamped_glu(const void* in, int in_dtype, void* out, int out_dtype, long rows, int F, float limit,
-                              float alpha, hipStream_t stream) {
+                              float alpha, float shift, hipStream_t stream) {
   GS_REQUIRE(rows >= 0 && F > 0, "clamped_glu: bad sizes rows=%ld F=%d", rows, F);
   if (rows == 0) return 0;
   const long total = rows * F;
   const int blocks = gs_ceil_div(total, 256);
   if (in_dtype == GS_F32 && out_dtype == GS_F32)
-    clamped_glu_kernel<float, float><<<blocks, 256, 0, stream>>>((const float*)in, (float*)out, F, total, limit, alpha);
+    clamped_glu_kernel<float, float><<<blocks, 256, 0, stream>>>((const float*)in, (float*)out, F, total, limit, alpha, shift);
   else if (in_dtype == GS_BF16 && out_dtype == GS_BF16)
-    clamped_glu_kernel<bf16, bf16><<<blocks, 256, 0, stream>>>((const bf16*)in, (bf16*)out, F, total, limit, alpha);
+    clamped_glu_kernel<bf16, bf16><<<blocks, 256, 0, stream>>>((const bf16*)in, (bf16*)out, F, total, limit, alpha, shift);
   else if (in_dtype == GS_F32 && out_dtype == GS_BF16)
-    clamped_glu_kernel<float, bf16><<<blocks, 256, 0, stream>>>((const float*)in, (bf16*)out, F, total, limit, alpha);
+    clamped_glu_kernel<float, bf16><<<blocks, 256, 0, stream>>>((const float*)in, (bf16*)out, F, total, limit, alpha, shift);
   else
     GS_REQUIRE(false, "clamped_glu: unsupported types %d %d", in_dtype, out_dtype);
   GS_LAUNCH_CHECK("clamped_glu");
@@ -344,7 +346,7 @@ extern "C" int gs_clamped_glu(const void* in, int in_dtype, void* out, int out_d
 }
 
 extern "C" int gs_moe_routed_up(const void* x, int dtype, int ldx, const int* choice, int top, int E, const void* gate_up,
-                                int w_dtype, int F, int H, float limit, float alpha, void* a, int ntok,
+                                int w_dtype, int F, int H, float limit, float alpha, float shift, void* a, int ntok,
                                 hipStream_t stream) {
   GS_REQUIRE(ntok >= 0 && top > 0 && F > 0 && H > 0 && ldx >= H && E >= 0, "moe_routed_up: bad sizes T=%d top=%d F=%d H=%d", ntok, top, F, H);
   GS_REQUIRE(H * sizeof(float) <= 65536, "moe_routed_up: rows of %d are wider than the kernel's staging", H);
@@ -353,7 +355,7 @@ extern "C" int gs_moe_routed_up(const void* x, int dtype, int ldx, const int* ch
   const size_t lds = H * sizeof(float);
 #define GS_RUN(T, TW)                                                                                                 \
   moe_routed_up_kernel<T, TW><<<grid, 256, lds, stream>>>((const T*)x, ldx, choice, top, E, (const TW*)gate_up, F, H, \
-                                                          limit, alpha, (T*)a)
+                                                          limit, alpha, shift, (T*)a)
   if (dtype == GS_F32 && w_dtype == GS_F32)
     GS_RUN(float, float);
   else if (dtype == GS_BF16 && w_dtype == GS_BF16)

@@ -16,6 +16,9 @@
 // `plain_norm`: q and k are divided by their root mean square without a weight (a turn keeps a head's sum of squares,
 // so the same numbers come out whether the division stands before or after it).  `v_first` (rows `ldf` apart, the value
 // heads from column 0 on) with `mix` (one float on the device): the values are cached as (1 - mix) v + mix v_first.
+// `maps` > 1: a value head goes with that many keys of width d (the rows hold nkv maps key heads before the nkv value heads,
+// key head by key head, its maps side by side); the key cache is (num_pages, nkv, page_size, maps d), a head's keys of a
+// token side by side.
 // One wave per (token, head).  All arithmetic float32.
 #include "common.h"
 
@@ -28,30 +31,35 @@ __global__ void qknorm_rope_kv_kernel(T* __restrict__ qkv, const float* __restri
                                       int ntok, int nh, int nkv, int d, int write_kv, int vd,
                                       const float* __restrict__ vcos, const float* __restrict__ vsin, int ld,
                                       int plain_norm, const T* __restrict__ v_first, int ldf,
-                                      const float* __restrict__ mix) {
+                                      const float* __restrict__ mix, int maps) {
   int lane = threadIdx.x & 63;
-  int heads = nh + 2 * nkv;
+  const int nk = nkv * maps;
+  int heads = nh + nk + nkv;
   long unit = (long)blockIdx.x * (blockDim.x >> 6) + (threadIdx.x >> 6);
   if (unit >= (long)ntok * heads) return;
   int t = (int)(unit / heads);
   int hh = (int)(unit - (long)t * heads);
   const size_t row_len = (size_t)ld;
-  const bool is_v = hh >= nh + nkv;
-  T* x = qkv + (size_t)t * row_len + (is_v ? (size_t)(nh + nkv) * d + (size_t)(hh - nh - nkv) * vd : (size_t)hh * d);
+  const bool is_v = hh >= nh + nk;
+  T* x = qkv + (size_t)t * row_len + (is_v ? (size_t)(nh + nk) * d + (size_t)(hh - nh - nk) * vd : (size_t)hh * d);
   int pos = positions[t];
 
   T* dst = nullptr;  // cache row for k and v heads
   if (hh >= nh) {
     if (!write_kv) return;
-    int kvh = is_v ? hh - nh - nkv : hh - nh;
+    int kvh = is_v ? hh - nh - nk : hh - nh, map = 0;
+    if (!is_v && maps > 1) {
+      map = kvh % maps;
+      kvh /= maps;
+    }
     int page = block_table[(size_t)seq_of_token[t] * max_blocks + pos / page_size];
     T* base = is_v ? vcache : kcache;
-    dst = base + (((size_t)page * nkv + kvh) * page_size + pos % page_size) * (is_v ? vd : d);
+    dst = base + (((size_t)page * nkv + kvh) * page_size + pos % page_size) * (is_v ? vd : maps * d) + map * d;
   }
   if (is_v) {  // v: copy, blend with another layer's values, or turn by the position over the whole width
     if (v_first) {
       const float lam = mix[0];
-      const T* f = v_first + (size_t)t * ldf + (size_t)(hh - nh - nkv) * vd;
+      const T* f = v_first + (size_t)t * ldf + (size_t)(hh - nh - nk) * vd;
       for (int j = lane; j < vd; j += 64) dst[j] = from_f32<T>((1.f - lam) * to_f32(x[j]) + lam * to_f32(f[j]));
       return;
     }
@@ -165,8 +173,9 @@ extern "C" int gs_qknorm_rope_kv(void* qkv, int dtype, const float* qw, const fl
                                  int max_position, const int* positions, const int* seq_of_token, const int* block_table,
                                  int max_blocks, int page_size, void* kcache, void* vcache, int ntok, int nh, int nkv,
                                  int d, int write_kv, int vd, const float* vcos, const float* vsin, int ld,
-                                 int plain_norm, const void* v_first, int ldf, const float* mix,
+                                 int plain_norm, const void* v_first, int ldf, const float* mix, int maps,
                                  hipStream_t stream) {
+  GS_REQUIRE(maps >= 1 && maps <= 64, "qknorm_rope_kv: %d keys a head", maps);
   GS_REQUIRE(vd > 0, "qknorm_rope_kv: values of width %d", vd);
   GS_REQUIRE((vcos == nullptr) == (vsin == nullptr), "qknorm_rope_kv: the value tables come together");
   GS_REQUIRE(!vcos || (vd % 2 == 0 && max_position > 0), "qknorm_rope_kv: turned values are of even width");
@@ -178,15 +187,15 @@ extern "C" int gs_qknorm_rope_kv(void* qkv, int dtype, const float* qw, const fl
   GS_REQUIRE(page_size > 0 && max_blocks > 0, "qknorm_rope_kv: bad page_size %d or max_blocks %d", page_size,
              max_blocks);
   GS_REQUIRE((qw == nullptr) == (kw == nullptr), "qknorm_rope_kv: q and k norm weights come together");
-  const int narrow = (nh + nkv) * d + nkv * vd;
+  const int narrow = (nh + nkv * maps) * d + nkv * vd;
   if (ld == 0) ld = narrow;
   GS_REQUIRE(ld >= narrow, "qknorm_rope_kv: rows of %d values do not hold q, k and v (%d)", ld, narrow);
   GS_REQUIRE(!(plain_norm && qw), "qknorm_rope_kv: a head norm has a weight or none");
   GS_REQUIRE((v_first == nullptr) == (mix == nullptr) && (!v_first || (ldf >= nkv * vd && !vcos)),
              "qknorm_rope_kv: blended values need the other values (rows of at least %d) and the share", nkv * vd);
   if (ntok == 0) return 0;
-  long units = (long)ntok * (nh + 2 * nkv);
-  const bool vec = ld == narrow && !plain_norm && !v_first && !interleaved && vd == d && !vcos && rotary_dim == d && (d == 16 || d == 32 || d == 64 || d == 128) && (dtype == GS_F32 || dtype == GS_BF16) &&
+  long units = (long)ntok * (nh + nkv * maps + nkv);
+  const bool vec = maps == 1 && ld == narrow && !plain_norm && !v_first && !interleaved && vd == d && !vcos && rotary_dim == d && (d == 16 || d == 32 || d == 64 || d == 128) && (dtype == GS_F32 || dtype == GS_BF16) &&
                    ((uintptr_t)qkv & 15) == 0 && ((uintptr_t)kcache & 15) == 0 && ((uintptr_t)vcache & 15) == 0 &&
                    ((uintptr_t)cos_t & 15) == 0 && ((uintptr_t)sin_t & 15) == 0 && ((uintptr_t)qw & 15) == 0 &&
                    ((uintptr_t)kw & 15) == 0;
@@ -215,7 +224,7 @@ extern "C" int gs_qknorm_rope_kv(void* qkv, int dtype, const float* qw, const fl
   qknorm_rope_kv_kernel<T><<<blocks, 256, 0, stream>>>((T*)qkv, qw, kw, eps, cos_t, sin_t, rotary_dim, interleaved, positions, \
                                                        seq_of_token, block_table, max_blocks, page_size,        \
                                                        (T*)kcache, (T*)vcache, ntok, nh, nkv, d, write_kv, vd, vcos, vsin, \
-                                                       ld, plain_norm, (const T*)v_first, ldf, mix)
+                                                       ld, plain_norm, (const T*)v_first, ldf, mix, maps)
   if (dtype == GS_F32)
     GS_RUN(float);
   else if (dtype == GS_BF16)

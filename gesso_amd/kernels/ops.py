@@ -315,18 +315,20 @@ def _value_tables(vcos, vsin, vd):
 
 def qknorm_rope_kv(qkv, q_weight, k_weight, eps, cos, sin, rotary_dim, positions, seq_of_token, block_table,
                    page_size, kcache, vcache, nh, nkv, d, write_kv=True, layout: str = "half", vd: int = None,
-                   vcos=None, vsin=None, plain_norm: bool = False, v_first=None, mix=None) -> None:
+                   vcos=None, vsin=None, plain_norm: bool = False, v_first=None, mix=None, maps: int = 1) -> None:
     """Head norm and rotation of q (in place) and k; k and v written into the pages.  ``layout``: which features
     form a rotation pair, ``"half"`` (i, i + rotary_dim/2) or ``"interleaved"`` (2i, 2i + 1).  ``vd``: the width of
     a value head where it is not ``d``; ``vcos``, ``vsin`` ``(P, vd/2)``: the values are cached turned by their
     position over their whole width.  The rows may hold more columns behind q|k|v.  ``plain_norm``: q and k are divided
     by their root mean square, no weight.  ``v_first (T, >= nkv vd)`` (a range of columns of wider rows will do) with
-    ``mix`` (one float32 on the device): the values are cached as ``(1 - mix) v + mix v_first``."""
+    ``mix`` (one float32 on the device): the values are cached as ``(1 - mix) v + mix v_first``.  ``maps``: a value head
+    goes with that many keys of width ``d``, side by side in the rows and in the key cache ``(pages, nkv, page_size,
+    maps d)`` (``nh`` counts every query)."""
     _need(layout in ROPE_LAYOUTS, f"qknorm_rope_kv: pairs are laid out 'half' or 'interleaved', not {layout!r}")
     _dev(qkv, q_weight, k_weight, cos, sin, positions, seq_of_token, block_table, kcache, vcache, mix)
     vd = d if vd is None else int(vd)
     T = qkv.shape[0]
-    _need(qkv.dim() == 2 and qkv.shape[1] >= (nh + nkv) * d + nkv * vd, "qknorm_rope_kv: rows hold at least (nh + nkv) d + nkv vd values")
+    _need(qkv.dim() == 2 and qkv.shape[1] >= (nh + nkv * maps) * d + nkv * vd, "qknorm_rope_kv: rows hold at least (nh + nkv) d + nkv vd values")
     _need(not (plain_norm and q_weight is not None), "qknorm_rope_kv: a head norm has a weight or none")
     _need((v_first is None) == (mix is None), "qknorm_rope_kv: the other values and their share come together")
     ldf = 0
@@ -349,7 +351,7 @@ def qknorm_rope_kv(qkv, q_weight, k_weight, eps, cos, sin, rotary_dim, positions
     _i32(seq_of_token, T, "seq_of_token")
     _need(block_table.dtype == torch.int32 and block_table.dim() == 2, "block_table must be int32 (nseq, max_blocks)")
     _need(kcache.dtype == qkv.dtype and vcache.dtype == qkv.dtype, "cache and activations differ in type")
-    _need(kcache.dim() == 4 and kcache.shape[1:] == (nkv, page_size, d) and vcache.shape == kcache.shape[:3] + (vd,),
+    _need(kcache.dim() == 4 and kcache.shape[1:] == (nkv, page_size, maps * d) and vcache.shape == kcache.shape[:3] + (vd,),
           "caches must be (pages, nkv, page_size, d) and (pages, nkv, page_size, vd)")
     _check(lib().gs_qknorm_rope_kv(_p(qkv), c_int(_dt(qkv)), _p(q_weight), _p(k_weight), c_float(eps), _p(cos),
                                    _p(sin), c_int(rotary_dim), c_int(1 if layout == "interleaved" else 0), c_int(max_pos),
@@ -357,7 +359,7 @@ def qknorm_rope_kv(qkv, q_weight, k_weight, eps, cos, sin, rotary_dim, positions
                                    _p(block_table), c_int(block_table.shape[1]), c_int(page_size), _p(kcache),
                                    _p(vcache), c_int(T), c_int(nh), c_int(nkv), c_int(d),
                                    c_int(1 if write_kv else 0), c_int(vd), _p(vcos), _p(vsin), c_int(qkv.shape[1]),
-                                   c_int(1 if plain_norm else 0), _p(v_first), c_int(ldf), _p(mix), _stream()))
+                                   c_int(1 if plain_norm else 0), _p(v_first), c_int(ldf), _p(mix), maps, _stream()))
 
 
 def attention_generic(q, q_stride, kcache, vcache, positions, seq_of_token, block_table, page_size, window, scale,
@@ -395,11 +397,41 @@ def attention_generic(q, q_stride, kcache, vcache, positions, seq_of_token, bloc
     return out
 
 
+def _maps_operands(rows, kcache, vcache, positions, block_table, page_size, gate_col, nh, nkv, d, vd, what):
+    """The checks that the kernels of attention over two maps share."""
+    _dev(rows, kcache, vcache, positions, block_table)
+    _need(rows.dim() == 2 and rows.shape[1] >= 2 * nh * d and (gate_col < 0 or gate_col + nh <= rows.shape[1]),
+          f"{what}: rows hold 2 nh d query values and, from gate_col on, a gate a head")
+    _need(kcache.dtype == rows.dtype and vcache.dtype == rows.dtype, f"{what}: cache and activations differ in type")
+    _need(kcache.dim() == 4 and kcache.shape[1:] == (nkv, page_size, 2 * d) and vcache.shape == kcache.shape[:3] + (vd,),
+          f"{what}: caches must be (pages, nkv, page_size, 2 d) and (pages, nkv, page_size, vd)")
+    _need(block_table.dtype == torch.int32 and block_table.dim() == 2, "block_table must be int32 (nseq, max_blocks)")
+
+
+def attention_maps(rows, kcache, vcache, positions, seq_of_token, block_table, page_size, window, scale, lam: float, eps: float,
+                   out_scale: float, gate_col: int, nh, nkv, d, vd, out: torch.Tensor = None) -> torch.Tensor:
+    """The difference of two softmax maps over one value row, any sizes: query head ``h`` has its two queries at columns
+    ``[2 h d, (2 h + 2) d)`` of ``rows (T, ld)``, its key head two keys a token side by side in the cache;
+    ``o = o_1 - lam o_2`` per head, divided by its root mean square (``eps`` inside the root), times ``out_scale`` and, with
+    ``gate_col >= 0``, ``sigmoid(rows[:, gate_col + h])``.  Returns ``(T, nh vd)`` in the rows' type."""
+    T = rows.shape[0]
+    _maps_operands(rows, kcache, vcache, positions, block_table, page_size, gate_col, nh, nkv, d, vd, "attention_maps")
+    _i32(positions, T, "positions")
+    _i32(seq_of_token, T, "seq_of_token")
+    if out is None:
+        out = torch.empty((T, nh * vd), dtype=rows.dtype, device=rows.device)
+    _need(out.shape == (T, nh * vd) and out.dtype == rows.dtype and out.is_contiguous(), "attention_maps: out has the wrong shape or type")
+    _check(lib().gs_attention_maps(_p(rows), rows.shape[1], _p(kcache), _p(vcache), _dt(rows), _p(positions), _p(seq_of_token),
+                                   _p(block_table), block_table.shape[1], page_size, window or 0, scale, lam, eps, out_scale,
+                                   gate_col, _p(out), T, nh, nkv, d, vd, _stream()))
+    return out
+
+
 # ---------------------------------------------------------------------- linear attention
 
 _ACTS = {None: 0, "none": 0, "silu": 1}
 _GATES = {"sigmoid": 0, "silu": 1}
-GATED_ACTS = {"silu": 0, "gelu_tanh": 1}
+GATED_ACTS = {"silu": 0, "gelu_tanh": 1, "gelu": 2}
 LINEAR_ATTENTION_MAX_KEY = 512
 LINEAR_ATTENTION_CHUNKS_MAX_KEY = 128
 
@@ -469,8 +501,8 @@ def gated_outnorm(o, gate_rows, og: int, weight, eps: float, H: int, m: int, joi
     _dev(o, gate_rows, weight)
     T = o.shape[0]
     _need(o.dtype == torch.float32 and o.shape == (T, H * m), "gated_outnorm: o must be float32 (T, H m)")
-    _need(gate_rows.dim() == 2 and gate_rows.shape[0] == T and gate_rows.dtype == out_dtype,
-          "gated_outnorm: the gate's rows are (T, ldg) in the result's type")
+    _need(gate_rows.dim() == 2 and gate_rows.shape[0] == T and gate_rows.dtype in (out_dtype, torch.float32),
+          "gated_outnorm: the gate's rows are (T, ldg), float32 or in the result's type")
     _need(weight is None or (weight.dtype == torch.float32 and weight.shape == (H * m,)), "gated_outnorm: weight must be float32 (H m,)")
     _need(gate in _GATES, f"gated_outnorm: the gate is 'sigmoid' or 'silu', not {gate!r}")
     out = torch.empty((T, H * m), dtype=out_dtype, device=o.device)
@@ -521,6 +553,15 @@ def gated_act(x, bias, activation: str, out_dtype) -> torch.Tensor:
     out = torch.empty((T, F), dtype=out_dtype, device=x.device)
     _check(lib().gs_gated_act(_p(x), c_int(_dt(x)), _p(bias), _p(out), c_int(_dt(out)), c_int(T), c_int(F),
                               c_int(GATED_ACTS[activation]), _stream()))
+    return out
+
+
+def activate(x, activation: str, out_dtype) -> torch.Tensor:
+    """``act(x)`` elementwise in float32, rounded once to ``out_dtype``."""
+    _dev(x)
+    _need(activation in GATED_ACTS, f"activate: the activation is one of {sorted(GATED_ACTS)}, not {activation!r}")
+    out = torch.empty(x.shape, dtype=out_dtype, device=x.device)
+    _check(lib().gs_activate(_p(x), _dt(x), _p(out), _dt(out), x.numel(), GATED_ACTS[activation], _stream()))
     return out
 
 
@@ -1452,33 +1493,34 @@ def ssd_scan(xbc, rows, odt: int, dt_bias, a_log, d_skip, state, q_start, slots,
 ROUTER_SCORES = {"softmax": 0, "sigmoid": 1}
 
 
-def moe_router(x, router, correction, top: int, score: str = "softmax", renormalize: bool = True, scale: float = 1.0):
-    """Scores = softmax (or, with ``score="sigmoid"``, each output's sigmoid) of ``router (EA, H) @ x[t]`` in float32; the
+def moe_router(x, router, correction, top: int, score: str = "softmax", renormalize: bool = True, scale: float = 1.0, bias=None):
+    """Scores = softmax (or, with ``score="sigmoid"``, each output's sigmoid) of ``router (EA, H) @ x[t] (+ bias)`` in float32; the
     ``top`` outputs with the largest score + ``correction`` are chosen (of equal ones the lowest index), their weights
     are their scores divided by the chosen scores' sum (+ 1e-20) (as they are without ``renormalize``), times ``scale``.
     Returns ``(choice int32 (T, top), weight float32 (T, top))``."""
     _need(score in ROUTER_SCORES, f"moe_router: scores are one of {sorted(ROUTER_SCORES)}, not {score!r}")
-    _dev(router, correction)
+    _dev(router, correction, bias)
     ldx = _cols(x, "moe_router")
     T, H = x.shape
     EA = router.shape[0]
     _need(router.shape == (EA, H) and 1 <= top <= EA, "moe_router: the router is (outputs, H), top within its outputs")
     _need(correction is None or (correction.dtype == torch.float32 and correction.shape == (EA,)), "moe_router: the correction must be float32 (outputs,)")
+    _need(bias is None or (bias.dtype == torch.float32 and bias.shape == (EA,)), "moe_router: the bias must be float32 (outputs,)")
     choice = torch.empty((T, top), dtype=torch.int32, device=x.device)
     weight = torch.empty((T, top), dtype=torch.float32, device=x.device)
     _check(lib().gs_moe_router(_p(x), _dt(x), ldx, _p(router), _dt(router), _p(correction), top, EA, H, _p(choice),
-                               _p(weight), T, ROUTER_SCORES[score], 1 if renormalize else 0, float(scale), _stream()))
+                               _p(weight), T, ROUTER_SCORES[score], 1 if renormalize else 0, float(scale), _p(bias), _stream()))
     return choice, weight
 
 
-def clamped_glu(gu, limit: float, alpha: float, out_dtype) -> torch.Tensor:
-    """``gu (rows, 2F)`` = gate | up  ->  ``g sigmoid(alpha g) (u + 1)`` with ``g = min(gate, limit)``,
-    ``u = clamp(up, -limit, limit)``: ``(rows, F)`` in ``out_dtype``, float32 arithmetic."""
+def clamped_glu(gu, limit: float, alpha: float, out_dtype, shift: float = 1.0) -> torch.Tensor:
+    """``gu (rows, 2F)`` = gate | up  ->  ``g sigmoid(alpha g) (u + shift)`` with ``g = min(gate, limit)``,
+    ``u = clamp(up, -limit, limit)`` (``limit`` may be infinite): ``(rows, F)`` in ``out_dtype``, float32 arithmetic."""
     _dev(gu)
     _need(gu.dim() == 2 and gu.shape[1] % 2 == 0, "clamped_glu: rows hold gate and up side by side")
     R, F2 = gu.shape
     out = torch.empty((R, F2 // 2), dtype=out_dtype, device=gu.device)
-    _check(lib().gs_clamped_glu(_p(gu), _dt(gu), _p(out), _dt(out), R, F2 // 2, float(limit), float(alpha), _stream()))
+    _check(lib().gs_clamped_glu(_p(gu), _dt(gu), _p(out), _dt(out), R, F2 // 2, float(limit), float(alpha), float(shift), _stream()))
     return out
 
 
@@ -1495,7 +1537,7 @@ def _routed_operands(x, choice, weight, gate_up, down, shared, what):
     return ldx, T, H, E, F, choice.shape[1]
 
 
-def moe_routed(x, choice, weight, gate_up, down, limit: float, alpha: float, shared=None) -> torch.Tensor:
+def moe_routed(x, choice, weight, gate_up, down, limit: float, alpha: float, shared=None, shift: float = 1.0) -> torch.Tensor:
     """``y[t] = sum_k weight[t, k] * expert(choice[t, k])(x[t]) (+ shared[t])``, token by token: only the chosen experts'
     weights are read.  A choice ``>= E`` names no weights: that expert gives back ``x[t]``.  ``gate_up (E, 2F, H)`` holds
     each expert's gate rows, then its up rows; ``down (E, H, F)``."""
@@ -1503,7 +1545,7 @@ def moe_routed(x, choice, weight, gate_up, down, limit: float, alpha: float, sha
     a = torch.empty((T, top, max(F, 1)), dtype=x.dtype, device=x.device)
     y = torch.empty((T, H), dtype=x.dtype, device=x.device)
     _check(lib().gs_moe_routed_up(_p(x), _dt(x), ldx, _p(choice), top, E, _p(gate_up), _dt(gate_up), F, H, float(limit),
-                                  float(alpha), _p(a), T, _stream()))
+                                  float(alpha), float(shift), _p(a), T, _stream()))
     _check(lib().gs_moe_routed_down(_p(a), _dt(a), _p(x), ldx, _p(choice), _p(weight), top, E, _p(down), _dt(down), F, H,
                                     _p(shared), _p(y), T, _stream()))
     return y
@@ -1517,7 +1559,8 @@ def moe_routed_grouped_ok(x, gate_up, down) -> bool:
             and x.data_ptr() % 16 == 0 and 0 < down.shape[0] <= 4096)
 
 
-def moe_routed_grouped(x, choice, weight, gate_up, down, limit: float, alpha: float, shared=None) -> torch.Tensor:
+def moe_routed_grouped(x, choice, weight, gate_up, down, limit: float, alpha: float, shared=None,
+                       shift: float = 1.0) -> torch.Tensor:
     """:func:`moe_routed` for steps of many tokens (bfloat16): the (token, choice) pairs are sorted by expert on the
     device and every expert's weights are read once, by products on the matrix cores over its pairs' rows."""
     _need(moe_routed_grouped_ok(x, gate_up, down), "moe_routed_grouped: bfloat16 rows and weights, widths multiples of 8")
@@ -1535,7 +1578,7 @@ def moe_routed_grouped(x, choice, weight, gate_up, down, limit: float, alpha: fl
     _check(L.gs_moe_route(None, _p(choice), T, top, E, _p(perm), _p(place_of), _p(tiles), max_tiles, _p(n_tiles), s))
     _check(L.gs_moe_group_gemm(_p(x), ldx, _p(perm), _p(gate_up), _p(gu), BF16, 2 * F, _p(tiles), max_tiles, _p(n_tiles),
                                2 * F, H, 1, s))
-    inner = clamped_glu(gu, limit, alpha, torch.bfloat16)
+    inner = clamped_glu(gu, limit, alpha, torch.bfloat16, shift)
     _check(L.gs_moe_group_gemm(_p(inner), F, None, _p(down), _p(ys), F32, H, _p(tiles), max_tiles, _p(n_tiles), H, F, 0, s))
     _check(L.gs_moe_routed_combine(_p(ys), _p(place_of), _p(weight), top, _p(x), ldx, _p(shared), _p(y), _dt(y), T, H, s))
     return y
@@ -1673,20 +1716,28 @@ def gated_state_scan_segments(x, oq: int, ok: int, ov: int, H: int, qk_heads: in
     return gated_state_scan(x, oq, ok, ov, *args, m, decay, oa, per_channel, first, seg_start, ids, nseg, **kw)
 
 
-def delta_rule_prep(c, G: int, n: int, q_scale: float, unit_eps: float, rows, oa: int, ob: int, a_log, dt_bias, H: int):
+def delta_rule_prep(c, G: int, n: int, q_scale: float, unit_eps: float, rows, oa: int, ob: int, a_log, dt_bias, H: int,
+                    channels=None, oz: int = 0):
     """In place on ``c (T, >= 2 G n)`` float32: each of the ``G`` q heads (first) and ``G`` k heads (behind them) becomes
     ``x / sqrt(sum(x^2) + unit_eps)``, q also times ``q_scale``.  Returns float32 ``(T, 2 H)``:
     ``exp(-exp(a_log) softplus(rows[:, oa + h] + dt_bias))`` in the first ``H`` columns, ``sigmoid(rows[:, ob + h])`` in
-    the others."""
-    _dev(c, rows, a_log, dt_bias)
+    the others.
+
+    ``channels (T, ldz)`` float32: a decay a head and key channel instead, in place in its columns ``[oz, oz + H n)``:
+    ``z <- exp(-exp(a_log[h]) softplus(z + dt_bias))`` with ``dt_bias (H n,)``; the result is then ``beta`` alone ``(T, H)``."""
+    _dev(c, rows, a_log, dt_bias, channels)
     T = c.shape[0]
     _need(c.dtype == torch.float32 and c.dim() == 2 and c.shape[1] >= 2 * G * n, "delta_rule_prep: float32 rows that hold q and k")
     _need(rows.dim() == 2 and rows.shape[0] == T, "delta_rule_prep: the gates' products are rows (T, ld)")
-    for v in (a_log, dt_bias):
-        _need(v.dtype == torch.float32 and v.shape == (H,), "delta_rule_prep: a_log and dt_bias must be float32 (H,)")
-    gates = torch.empty((T, 2 * H), dtype=torch.float32, device=c.device)
+    _need(a_log.dtype == torch.float32 and a_log.shape == (H,), "delta_rule_prep: a_log must be float32 (H,)")
+    _need(dt_bias.dtype == torch.float32 and dt_bias.shape == (H if channels is None else H * n,),
+          "delta_rule_prep: dt_bias must be float32 (H,), or (H n,) with a decay a channel")
+    _need(channels is None or (channels.dtype == torch.float32 and channels.dim() == 2 and channels.shape[0] == T),
+          "delta_rule_prep: the channels' products are float32 rows (T, ldz)")
+    gates = torch.empty((T, 2 * H if channels is None else H), dtype=torch.float32, device=c.device)
     _check(lib().gs_delta_rule_prep(_p(c), c.shape[1], G, n, float(q_scale), float(unit_eps), _p(rows), _dt(rows),
-                                    rows.shape[1], oa, ob, _p(a_log), _p(dt_bias), _p(gates), T, H, _stream()))
+                                    rows.shape[1], oa, ob, _p(a_log), _p(dt_bias), _p(gates), T, H, _p(channels),
+                                    0 if channels is None else channels.shape[1], oz, _stream()))
     return gates
 
 

@@ -36,7 +36,8 @@ def tensor_table(spec: ModelSpec) -> Dict[str, TensorSpec]:
     if not spec.tie_embeddings:
         put(spec.names["head"], TensorSpec((spec.vocab, spec.hidden), MATRIX))
     if spec.reentry is not None:
-        put(spec.names["reentry.weight"], TensorSpec((spec.hidden, 2 * spec.hidden), MATRIX))
+        if spec.reentry.mix:
+            put(spec.names["reentry.weight"], TensorSpec((spec.hidden, 2 * spec.hidden), MATRIX))
         put(spec.names["reentry.step"], TensorSpec((len(spec.reentry.at), spec.hidden), VECTOR))
     for i, b in enumerate(spec.blocks):
         for local, ts in part_class("block", b).tensor_specs(b).items():
@@ -83,7 +84,8 @@ class Model:
             self.embed_norm.bind({k: tensors[s.names["embed_norm." + k]]
                                   for k in part_class("norm", s.embed_norm).tensor_specs(s.embed_norm)})
         if s.reentry is not None:
-            self.reentry_weight = self.rt.prepare(tensors[s.names["reentry.weight"]])
+            if s.reentry.mix:
+                self.reentry_weight = self.rt.prepare(tensors[s.names["reentry.weight"]])
             self.reentry_step = tensors[s.names["reentry.step"]].contiguous()
         for b, block in zip(s.blocks, self.blocks):
             local = {k: tensors[b.names[k]] for k in part_class("block", b).tensor_specs(b)}
@@ -117,7 +119,7 @@ class Model:
         reentries = {} if self.spec.reentry is None else {at: t for t, at in enumerate(self.spec.reentry.at)}
         # the embedding output, kept for every re-entry of this step (in the activation type: it is a product's operand
         # from here on)
-        x0 = stream.res.to(rt.dtype, copy=True) if reentries else None
+        x0 = stream.res.to(rt.dtype, copy=True) if reentries and self.spec.reentry.mix else None
         for i, call in enumerate(self.spec.schedule):
             if i in reentries:
                 with rt.stage("reentry"):
@@ -128,8 +130,14 @@ class Model:
 
     def _reenter(self, stream: ResidualStream, x0, t: int) -> ResidualStream:
         """``x <- W [x; x0] + step[t]``: the stream and the embedding output side by side through one product, float32
-        sums, the pass's vector added in float32; the result is the new stream."""
+        sums, the pass's vector added in float32; the result is the new stream.  Without the product the vector is left
+        beside the stream, for the norm that reads it next to add."""
         rt = self.rt
+        if not self.spec.reentry.mix:
+            if stream.bias is not None:
+                stream.flush(rt)
+            stream.bias = self.reentry_step[t]
+            return stream
         stream.flush(rt)
         T, W = stream.res.shape
         rows = torch.empty((T, 2 * W), dtype=rt.dtype, device=stream.res.device)

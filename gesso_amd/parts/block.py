@@ -215,7 +215,7 @@ class SharedNormBlock(Part):
     def forward(self, stream, ctx, cache):
         rt, ops, s = self.rt, self.rt.ops, self.spec
         with rt.stage("norm"):
-            a = self.norm.add_norm(stream)
+            a = rt.dense(self.norm.add_norm(stream))
         x = a
         mixer_cache = cache
         if s.input_taps is not None:

@@ -15,7 +15,11 @@ from the walk in one piece by float32 rounding.
     S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
     out = W_o (rms(o) * w * silu(z))                 the norm per head, its weight shared by the heads
 
-The convolutions' last ``taps - 1`` inputs belong to the request's state too.
+The convolutions' last ``taps - 1`` inputs belong to the request's state too.  A spec may ask for a decay per head and key
+channel, ``g = exp(-exp(A_log_h) softplus(W_up (W_down x) + dt_bias))`` (``decay_rank`` features between the two products;
+it acts on the state's rows), for a gate through a bottleneck, ``z = W_up (W_down x)`` (``gate_rank``), and for the sigmoid
+in silu's place.  The bottlenecks' first products ride in the one input product; what lies behind them is one product of
+the two bottlenecks side by side, with zeros where one's features meet the other's outputs.
 
 ``GatedLinear`` (linear attention with a decay per key channel):
 
@@ -45,7 +49,7 @@ def _scan(ops, ctx, args, state, **kw):
     return ops.gated_state_scan(*args, state, ctx.q_start, ctx.slots, ctx.nseq, **kw)
 
 
-def _stacked(ws, pad_to: int = 16):
+def stacked(ws, pad_to: int = 16):
     """The weights one above the other, with rows of zeros below so that the row count is a multiple of ``pad_to``."""
     if len({w.dtype for w in ws}) > 1:
         ws = [w.float() for w in ws]
@@ -74,13 +78,19 @@ class GatedDelta(Part):
     @staticmethod
     def tensor_specs(spec):
         W, H, G, n, m, K = spec.hidden, spec.n_heads, spec.qk_heads, spec.key_dim, spec.value_dim, spec.conv_taps
-        return {"q_proj.weight": TensorSpec((G * n, W), MATRIX), "k_proj.weight": TensorSpec((G * n, W), MATRIX),
-                "v_proj.weight": TensorSpec((H * m, W), MATRIX), "gate_proj.weight": TensorSpec((H * m, W), MATRIX),
-                "beta_proj.weight": TensorSpec((H, W), MATRIX), "decay_proj.weight": TensorSpec((H, W), MATRIX),
-                "q_conv.weight": TensorSpec((G * n, K), VECTOR), "k_conv.weight": TensorSpec((G * n, K), VECTOR),
-                "v_conv.weight": TensorSpec((H * m, K), VECTOR), "A_log": TensorSpec((H,), VECTOR),
-                "dt_bias": TensorSpec((H,), VECTOR), "out_norm.weight": TensorSpec((m,), VECTOR, "one_plus_normal"),
-                "out_proj.weight": TensorSpec((W, H * m), MATRIX)}
+        out = {"q_proj.weight": TensorSpec((G * n, W), MATRIX), "k_proj.weight": TensorSpec((G * n, W), MATRIX),
+               "v_proj.weight": TensorSpec((H * m, W), MATRIX), "beta_proj.weight": TensorSpec((H, W), MATRIX),
+               "q_conv.weight": TensorSpec((G * n, K), VECTOR), "k_conv.weight": TensorSpec((G * n, K), VECTOR),
+               "v_conv.weight": TensorSpec((H * m, K), VECTOR), "A_log": TensorSpec((H,), VECTOR),
+               "out_norm.weight": TensorSpec((m,), VECTOR, "one_plus_normal"), "out_proj.weight": TensorSpec((W, H * m), MATRIX)}
+        for name, rank, rows in (("decay", spec.decay_rank, H if spec.decay_rank is None else H * n), ("gate", spec.gate_rank, H * m)):
+            if rank is None:
+                out[f"{name}_proj.weight"] = TensorSpec((rows, W), MATRIX)
+            else:
+                out[f"{name}_down.weight"] = TensorSpec((rank, W), MATRIX)
+                out[f"{name}_up.weight"] = TensorSpec((rows, rank), MATRIX)
+        out["dt_bias"] = TensorSpec((H if spec.decay_rank is None else H * n,), VECTOR)
+        return out
 
     @staticmethod
     def cache_need(spec):
@@ -90,7 +100,30 @@ class GatedDelta(Part):
 
     def bind(self, tensors):
         rt, s = self.rt, self.spec
-        self.w_in = rt.prepare(_stacked([tensors[k + "_proj.weight"] for k in ("q", "k", "v", "gate", "beta", "decay")]))
+        # the input product's rows: q | k | v | z | beta | a, then (from a multiple of 16 on) each bottleneck's features, in
+        # whole runs of 32 with rows of zeros behind them
+        whole = [k for k in ("gate", "beta", "decay") if k == "beta" or getattr(s, k + "_rank") is None]
+        parts = [stacked([tensors[k + "_proj.weight"] for k in ("q", "k", "v", *whole)])]
+        self.columns, at = {}, self.channels(s)
+        for k in whole:
+            self.columns[k] = at
+            at += tensors[k + "_proj.weight"].shape[0]
+        low = [k for k in ("decay", "gate") if getattr(s, k + "_rank") is not None]
+        downs = [stacked([tensors[k + "_down.weight"]], 32) for k in low]
+        self.low_at, self.low_width = parts[0].shape[0], sum(w.shape[0] for w in downs)
+        self.w_in = rt.prepare(stacked(parts + downs))
+        self.w_up, self.up_columns = None, {}
+        if low:
+            ups = [tensors[k + "_up.weight"] for k in low]
+            if len({w.dtype for w in ups}) > 1:
+                ups = [w.float() for w in ups]
+            up = torch.zeros((-(-sum(w.shape[0] for w in ups) // 16) * 16, self.low_width), dtype=ups[0].dtype, device=ups[0].device)
+            r = c = 0
+            for k, w, dn in zip(low, ups, downs):
+                self.up_columns[k] = r
+                up[r:r + w.shape[0], c:c + w.shape[1]] = w
+                r, c = r + w.shape[0], c + dn.shape[0]
+            self.w_up = rt.prepare(up)
         self.w_out = rt.prepare(tensors["out_proj.weight"])
         self.taps = torch.cat([tensors[k + "_conv.weight"] for k in ("q", "k", "v")], 0).contiguous()
         self.a_log, self.dt_bias = tensors["A_log"], tensors["dt_bias"]
@@ -102,17 +135,25 @@ class GatedDelta(Part):
         s, rt, ops = self.spec, self.rt, self.rt.ops
         H, G, n, m = s.n_heads, s.qk_heads, s.key_dim, s.value_dim
         C = self.channels(s)
+        per_channel = s.decay_rank is not None
         with rt.stage("delta_in"):
-            rows = rt.linear(rt.dense(x), self.w_in)                  # q | k | v | z | b | a (| spare columns)
+            rows = rt.linear(rt.dense(x), self.w_in)                  # q | k | v | z | b | a | bottlenecks (| spare columns)
+            ups = None
+            if self.w_up is not None:
+                ups = rt.linear(rows[:, self.low_at:self.low_at + self.low_width], self.w_up, out_dtype=torch.float32)
         with rt.stage("delta_conv"):
             qkv = ops.channel_conv(rows[:, :C], self.taps, None, cache.state["conv_history"], ctx.seq_of_token,
                                    ctx.q_start, ctx.slots, ctx.nseq, ctx.all_single, torch.float32, activation="silu")
-            gates = ops.delta_rule_prep(qkv, G, n, float(n) ** -0.5, s.unit_eps, rows, C + H * m + H, C + H * m,
-                                        self.a_log, self.dt_bias, H)
+            gates = ops.delta_rule_prep(qkv, G, n, float(n) ** -0.5, s.unit_eps, rows, self.columns.get("decay", 0),
+                                        self.columns["beta"], self.a_log, self.dt_bias, H,
+                                        channels=ups if per_channel else None, oz=self.up_columns.get("decay", 0))
         with rt.stage("delta_state"):
-            o = _scan(ops, ctx, (qkv, 0, G * n, 2 * G * n, H, G, n, m, gates, 0, False), cache.state["state"], beta=gates, ob=H)
+            decays, oa, ob = (ups, self.up_columns["decay"], 0) if per_channel else (gates, 0, H)
+            o = _scan(ops, ctx, (qkv, 0, G * n, 2 * G * n, H, G, n, m, decays, oa, per_channel), cache.state["state"],
+                      beta=gates, ob=ob)
         with rt.stage("delta_norm"):
-            y = ops.gated_outnorm(o, rows, C, self.norm_weight, s.eps, H, m, False, "silu", rt.dtype)
+            z, oz = (rows, self.columns["gate"]) if s.gate_rank is None else (ups, self.up_columns["gate"])
+            y = ops.gated_outnorm(o, z, oz, self.norm_weight, s.eps, H, m, False, s.gate, rt.dtype)
         return rt.linear(y, self.w_out, out_dtype=out_dtype)
 
 
@@ -142,8 +183,8 @@ class GatedLinear(Part):
 
     def bind(self, tensors):
         rt, s = self.rt, self.spec
-        self.w_in = rt.prepare(_stacked([tensors[k + "_proj.weight"] for k in ("q", "k", "v", "gate")]))
-        self.w_down = rt.prepare(_stacked([tensors["decay_down.weight"]]))
+        self.w_in = rt.prepare(stacked([tensors[k + "_proj.weight"] for k in ("q", "k", "v", "gate")]))
+        self.w_down = rt.prepare(stacked([tensors["decay_down.weight"]]))
         up = tensors["decay_up.weight"]
         spare = self.w_down.shape[0] - up.shape[1]                     # the bottleneck's spare rows are zeros: columns of
         if spare:                                                      # zeros here change no sum

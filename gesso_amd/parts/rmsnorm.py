@@ -111,6 +111,13 @@ class RMSNorm(Part):
         follows, which norms on the fly.
         """
         if isinstance(stream.pending, tuple) or stream.bias is not None:
+            held = stream.pending if isinstance(stream.pending, tuple) else (stream.pending, None)
+            if rows is None and out is None and len(held) == 2 and len({d.dtype for d in held if d is not None}) <= 1:
+                # what a block with two results left, and a vector for every row: added in the norm's own pass
+                y, _ = self.rt.ops.add_rmsnorm_pair(stream.res, held[0], held[1], self.weight, None, self.spec.eps,
+                                                    out_dtype or self.rt.dtype, bias=stream.bias)
+                stream.pending = stream.ssq = stream.xs = stream.xs_for = stream.normed = stream.rows = stream.bias = None
+                return y
             stream.flush(self.rt)
         if self.rt.fused and rows is None and stream.pending is None and stream.ssq is not None:
             mine = stream.xs_for is self

@@ -1,9 +1,10 @@
 """A mixture of gated feed-forwards chosen by a router over the token's features.
 
-    z = W_r x  (float32),  s = softmax(z) over all ``E + I`` router outputs  (``score = "sigmoid"``: s = sigmoid(z))
+    z = W_r x (+ b)  (float32),  s = softmax(z) over all ``E + I`` router outputs  (``score = "sigmoid"``: s = sigmoid(z))
     chosen: the ``top`` outputs with the largest ``s + correction``;  weights: ``s`` of the chosen / (their sum + 1e-20)
     (``renormalize = False``: ``s`` of the chosen as they are), times ``route_scale``
-    expert e < E:   W_down[e] (g sigmoid(alpha g) (u + 1)),  g = min(W_gate[e] x, limit),  u = clamp(W_up[e] x, -limit, limit)
+    expert e < E:   W_down[e] (g sigmoid(alpha g) (u + shift)),  g = min(W_gate[e] x, limit),  u = clamp(W_up[e] x, -limit, limit)
+                    (no limit: nothing is clamped)
     expert e >= E:  x itself (an identity expert: it has no tensors)
     y = sum over the chosen of weight * expert(x)  +  shared(x)   (an expert of its own width and limit, for every token)
 
@@ -11,6 +12,8 @@ The experts' weights are stacked at load, gate over up: ``(E, 2F, H)`` and ``(E,
 up rows are laid side by side, so one product gives both.  Router, softmax, choice and weights are float32.
 """
 from __future__ import annotations
+
+import math
 
 import torch
 
@@ -28,6 +31,8 @@ class RoutedMoE(Part):
         out = {"router.weight": TensorSpec((EA, H), MATRIX)}
         if spec.correction:
             out["router.correction"] = TensorSpec((EA,), VECTOR)
+        if getattr(spec, "router_bias", False):
+            out["router.bias"] = TensorSpec((EA,), VECTOR)
         for e in range(spec.n_experts):
             out[f"experts.{e}.gate.weight"] = TensorSpec((F, H), MATRIX)
             out[f"experts.{e}.up.weight"] = TensorSpec((F, H), MATRIX)
@@ -42,6 +47,9 @@ class RoutedMoE(Part):
         s, rt = self.spec, self.rt
         router = self.router = tensors["router.weight"].contiguous()
         self.correction = tensors.get("router.correction")
+        self.router_bias = tensors.get("router.bias")
+        self.limit = math.inf if s.limit is None else s.limit
+        self.shift = getattr(s, "shift", 1.0)
         E = s.n_experts
         gus = [torch.cat([tensors[f"experts.{e}.gate.weight"], tensors[f"experts.{e}.up.weight"]], 0) for e in range(E)]
         downs = [tensors[f"experts.{e}.down.weight"] for e in range(E)]
@@ -64,18 +72,18 @@ class RoutedMoE(Part):
         with rt.stage("ffn_router"):
             choice, weight = ops.moe_router(x, self.router, self.correction, s.top, score=getattr(s, "score", "softmax"),
                                             renormalize=getattr(s, "renormalize", True),
-                                            scale=getattr(s, "route_scale", 1.0))
+                                            scale=getattr(s, "route_scale", 1.0), bias=self.router_bias)
         shared = None
         if self.w_sgu is not None:
             with rt.stage("ffn_shared"):
-                limit = s.limit if s.shared_limit is None else s.shared_limit
-                shared = rt.linear(ops.clamped_glu(rt.linear(x, self.w_sgu), limit, s.alpha, rt.dtype), self.w_sdown)
+                limit = self.limit if s.shared_limit is None else s.shared_limit
+                shared = rt.linear(ops.clamped_glu(rt.linear(x, self.w_sgu), limit, s.alpha, rt.dtype, self.shift), self.w_sdown)
         # once the pairs outnumber the experts twice over, sorting them by expert reads less: each expert's weights
         # once, instead of once a pair (the option "token" keeps the token-by-token kernels for every step)
         if (x.shape[0] * s.top >= 2 * s.n_experts and rt.options.routed_experts != "token"
                 and ops.moe_routed_grouped_ok(x, self.gate_up, self.down)):
-            return ops.moe_routed_grouped(x, choice, weight, self.gate_up, self.down, s.limit, s.alpha, shared=shared)
-        return ops.moe_routed(x, choice, weight, self.gate_up, self.down, s.limit, s.alpha, shared=shared)
+            return ops.moe_routed_grouped(x, choice, weight, self.gate_up, self.down, self.limit, s.alpha, shared=shared, shift=self.shift)
+        return ops.moe_routed(x, choice, weight, self.gate_up, self.down, self.limit, s.alpha, shared=shared, shift=self.shift)
 
 
 register("ffn", "routed_moe", RoutedMoE)
