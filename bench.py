@@ -557,6 +557,62 @@ def kuditar_workload(steps: int = 64, warmup: int = 8, sizes=("1024", "2048"), o
     return out
 
 
+BILOLIX_SIZES = {
+    # six layers of which the first two run twice (eight layer runs): the delta rule with a dense feed-forward, two-map
+    # attention with experts | linear attention with a dense feed-forward, the delta rule with experts, the delta rule with a
+    # dense feed-forward, two-map attention with experts; keys, values, states and experts as wide as Kuditar's of that name,
+    # the ungated feed-forward as many weights as Kuditar's gated one
+    "1024": dict(width=1024, attn=(8, 4, 64, 128), delta=(8, 4, 64, 128), fading=(8, 64, 128), rank=64, window=512, ff=6912,
+                 experts=16, top=2, eff=512, vocab=65536, beside="1024"),
+    "2048": dict(width=2048, attn=(16, 4, 64, 128), delta=(16, 8, 64, 128), fading=(16, 64, 128), rank=128, window=1024, ff=12288,
+                 experts=32, top=4, eff=704, vocab=65536, beside="2048"),
+}
+
+
+def bilolix_config(size: str, max_position: int = 4096):
+    from gesso_amd.config import (BilolixConfig, BilolixLayer, ChannelDeltaConfig, FadingConfig, GeluFFConfig, LoopConfig,
+                                  MapAttentionConfig, PairTurn, SoftmaxMoEConfig)
+    z = BILOLIX_SIZES[size]
+    h, g, d, vd = z["attn"]
+    dense, moe = GeluFFConfig(z["ff"]), SoftmaxMoEConfig(z["experts"], z["top"], z["eff"])
+    attn = MapAttentionConfig(h, g, d, vd, d ** -0.5, 0.4, PairTurn(1e6, d), z["window"])
+    delta = ChannelDeltaConfig(*z["delta"], 4, z["rank"], z["rank"])
+    fading = FadingConfig(*z["fading"], 16.0, 16)
+    layers = (BilolixLayer("channel_delta", delta, dense), BilolixLayer("attention", attn, moe), BilolixLayer("gla", fading, dense),
+              BilolixLayer("channel_delta", delta, moe), BilolixLayer("channel_delta", delta, dense), BilolixLayer("attention", attn, moe))
+    return BilolixConfig(vocab=z["vocab"], width=z["width"], layers=layers, norm_eps=1e-6, loop=LoopConfig(0, 2, 2),
+                         max_position=max_position)
+
+
+def bilolix_workload(steps: int = 64, warmup: int = 8, sizes=("1024", "2048"), only: str = "", batches=(8, 64)) -> dict:
+    """Bilolix (attention over two maps, the delta rule and linear attention with channel decays, dense and routed
+    feed-forwards behind one norm a layer, a run of layers passed twice) at two sets of layer sizes, beside Kuditar of the
+    same width and as many layer runs: a 2,048-token prompt in one step, and decode steps at 512-token prompts."""
+    from gesso_amd import Engine
+    from gesso_amd.parts import RuntimeOptions
+    out = {"metric": "Bilolix beside Kuditar at equal width and depth: prefill and decode tok/s", "unit": "tok/s", "dtype": "bf16",
+           "data": "synthetic: uniform random token ids, random weights N(0, 0.02)", "sizes": {}}
+    for size in sizes:
+        row = {}
+        for name, cfg in (("bilolix", bilolix_config(size)), ("kuditar", kuditar_config(BILOLIX_SIZES[size]["beside"]))):
+            if only and only != name:
+                continue
+            engine = Engine.from_config(cfg, seed=0, dtype="bfloat16", page_size=16, max_context=4096,
+                                        max_tokens=max(batches) * (512 + steps + warmup + 32) + 4096, num_slots=max(batches) + 1,
+                                        options=RuntimeOptions(tune_library=True))
+            sec = prefill_run(engine, cfg, 2048)
+            r = {"prefill_tok_s": round(2048 / sec, 1), "prefill_ms": round(sec * 1e3, 3), "weights_gb": round(weight_bytes(engine) / 1e9, 3)}
+            for b in batches:
+                dt, _ = decode_run(engine, cfg, b, 512, steps, warmup, seed=40 + b)
+                r[f"decode_b{b}_tok_s"] = round(b * steps / dt, 1)
+                r[f"decode_b{b}_ms"] = round(dt / steps * 1e3, 4)
+            row[name] = r
+            del engine
+            torch.cuda.empty_cache()
+        out["sizes"][size] = row
+    return out
+
+
 def main() -> int:
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -576,7 +632,7 @@ def main() -> int:
     ap.add_argument("--launched-portions", action="store_true", help="launch the steps with prompt portions kernel by kernel instead of "
                     "replaying recordings of them (the prefill of the default line, --workload serve)")
     ap.add_argument("--token-budget", type=int, default=4096, help="--workload serve: the most tokens a step holds")
-    ap.add_argument("--workload", default="decode", choices=["decode", "serve", "long", "gemm", "stages", "makuzen", "fazezen", "togalorn", "kuditar"],
+    ap.add_argument("--workload", default="decode", choices=["decode", "serve", "long", "gemm", "stages", "makuzen", "fazezen", "togalorn", "kuditar", "bilolix"],
                     help="decode: the default line; serve: continuous batching at LFM2-350M sizes; long: LFM2-2.6B "
                          "sizes at a context of 32,768; gemm: the products of a 2,048-token prompt, ours beside the vendor's; "
                          "stages: the decode step stage by stage; makuzen: the Makuzen design at two sets of layer sizes "
@@ -587,6 +643,8 @@ def main() -> int:
     ap.add_argument("--togalorn-only", default="", choices=["", "togalorn", "makuzen"], help="--workload togalorn: one of the two models (for profiling)")
     ap.add_argument("--kuditar-sizes", default="1024,2048", help="--workload kuditar: which of its sizes")
     ap.add_argument("--kuditar-only", default="", choices=["", "kuditar", "fazezen"], help="--workload kuditar: one of the two models (for profiling)")
+    ap.add_argument("--bilolix-sizes", default="1024,2048", help="--workload bilolix: which of its sizes")
+    ap.add_argument("--bilolix-only", default="", choices=["", "bilolix", "kuditar"], help="--workload bilolix: one of the two models (for profiling)")
     ap.add_argument("--makuzen-sizes", default="1024,2048", help="--workload makuzen: which of its sizes")
     ap.add_argument("--makuzen-only", default="", choices=["", "makuzen", "lfm2"], help="--workload makuzen: one of the two models (for profiling)")
     args = ap.parse_args()
@@ -608,6 +666,10 @@ def main() -> int:
         if args.workload == "kuditar":
             print(json.dumps(kuditar_workload(min(args.steps, 64), min(args.warmup, 8), tuple(args.kuditar_sizes.split(",")),
                                               args.kuditar_only)))
+            return 0
+        if args.workload == "bilolix":
+            print(json.dumps(bilolix_workload(min(args.steps, 64), min(args.warmup, 8), tuple(args.bilolix_sizes.split(",")),
+                                              args.bilolix_only)))
             return 0
         if args.workload == "togalorn":
             print(json.dumps(togalorn_workload(min(args.steps, 64), min(args.warmup, 8), tuple(args.togalorn_sizes.split(",")),

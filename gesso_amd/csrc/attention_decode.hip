@@ -24,420 +24,13 @@
 // Everything that changes between steps (positions, block table) is read from device memory, so the
 // launch can be recorded into a graph.  q (T, q_stride), head h at [h D, (h+1) D); caches
 // (pages, nkv, page_size, D); out (T, nh D).  Window: keys lo..pos with lo = pos - window + 1.
-#include "common.h"
+#include "attention_decode_impl.h"
 #include "no_alloc.h"
 #include <mutex>
-
-#define DEC_MAXG 8
-#define DEC_LOG2E 1.4426950408889634f
-
-typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8_t;
-typedef __attribute__((ext_vector_type(4))) float f32x4_t;
-
-// With RAW, q points at rows of q|k|v as their product left them (q heads, then k heads, then v heads), and the
-// kernel does what comes between that product and attention itself: the head norms of q and k, the rotation, and
-// the write of the new key and value into their page.  Every block norms and rotates its own queries; the block
-// whose keys end with the new one norms and rotates it, keeps it and the value in LDS for its scores, and writes
-// both to the cache for the steps to come.  Heads of 64 or 128, rotated whole.
-// Where column c of sequence seq's output goes: a row of `width`, or tiled rows (out_tiles = ceil(nseq / 16) > 0),
-// the order in which the product that follows takes them.
-__device__ __forceinline__ size_t out_index(int seq, int c, int width, int out_tiles) {
-  return out_tiles ? tiled_index(seq, c, out_tiles) : (size_t)seq * width + c;
-}
-
-struct DecodeRaw {
-  const float* qw;       // (D) head norm weights, or null for no norm
-  const float* kw;
-  float eps;
-  const float* cos_t;    // (positions, D / 2)
-  const float* sin_t;
-  int write_kv;          // 0: another layer owns the cache; the new key is already in it
-  // (read with and without RAW) chunk > 0: the query sees no key before the first position of its own run of `chunk`
-  // positions; sink: one more term exp(0), without a value, in the softmax's denominator
-  int chunk;
-  int sink;
-  // softcap > 0: a score becomes softcap tanh(score / softcap).  keep_first > 0 (with a window, without runs): the
-  // sequence's first keep_first positions stay visible when the window has passed them.  sinks (one float32 a head):
-  // the extra term of the denominator is exp(sinks[h]) instead of exp(0).
-  float softcap;
-  int keep_first;
-  const float* sinks;
-};
-
-template <int D, int G, int W, int RAW>
-__global__ __launch_bounds__(W * 64) void attention_decode_kernel(
-    const bf16* __restrict__ q, int q_stride, bf16* kcache, bf16* vcache,
-    const int* __restrict__ positions, const int* __restrict__ block_table, int max_blocks, int page_size,
-    unsigned page_magic, int window, float scale, bf16* __restrict__ out, float* __restrict__ part_o,
-    float* __restrict__ part_ml, int nh, int nkv, int out_tiles, DecodeRaw raw) {
-  static_assert(!RAW || D == 64 || D == 128, "the fused head norm and rotation are written for heads of 64 and 128");
-  constexpr int DC = D / 8;               // 16-byte chunks per row
-  constexpr int KG = 64 / DC;             // key groups per wavefront in the value phase
-  constexpr int NI = 64 / KG;             // keys per lane in the value phase
-  constexpr int KS = (D + 31) / 32;       // steps of 32 features in the score products
-  static_assert(D % 8 == 0 && 64 % DC == 0 && G <= 16, "head width must be 8, 16, 32, 64, 128, 256 or 512");
-  // What the registers allow (256 a lane at eight wavefronts a block): the next tile's rows in flight while
-  // this one is computed, for rows of up to 64.
-  constexpr bool PIPE = D <= 64;
-  __shared__ float ps[W][G][64];          // a tile's probabilities, then read per key in the value phase
-  __shared__ float al[W][G];              // by how much a tile shrinks what was accumulated before it
-  __shared__ float wm[W][G], wl[W][G];
-  __shared__ float wacc[W][G][D];
-
-  const int split = blockIdx.x, nsplit = gridDim.x, kvh = blockIdx.y, seq = blockIdx.z;
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-  const int r16 = lane & 15, kg = lane >> 4;
-  const int pos = positions[seq];
-  int lo_real = window > 0 ? (pos - window + 1 > 0 ? pos - window + 1 : 0) : 0;
-  if (raw.chunk > 0 && pos - pos % raw.chunk > lo_real) lo_real = pos - pos % raw.chunk;
-  // The kept first positions that the window has passed stand before the window's keys in one row of places: place
-  // lo + i is key i for the `kept` first places, and key lo + i (itself) from there on.
-  const int kept = (raw.keep_first > 0 && window > 0 && raw.chunk == 0) ? (raw.keep_first < lo_real ? raw.keep_first : lo_real) : 0;
-  const int lo = lo_real - kept;
-  const int nkeys = pos - lo + 1;
-  // this block's share of the keys, in whole tiles of 64
-  const int tiles = (nkeys + 63) >> 6;
-  const int tper = (tiles + nsplit - 1) / nsplit;
-  const int t0 = split * tper, t1 = (t0 + tper < tiles) ? t0 + tper : tiles;
-  const int* bt = block_table + (size_t)seq * max_blocks;
-  const int dc = lane % DC, kq = lane / DC;
-
-  // where key u's row starts in the caches (u <= pos)
-  // (u / page_size as one multiplication, page_magic = floor(2^32 / page_size) + 1, exact while u page_size < 2^32:
-  // no branch near the loads, which would make the compiler wait for every load in flight)
-  auto row_off = [&](int u) -> long {
-    u = u < lo_real ? u - lo : u;          // a place before the window's first key holds a kept first position
-    const int pg = (int)__umulhi((unsigned)u, page_magic);
-    const int r = u - pg * page_size;
-    return (((long)bt[pg] * nkv + kvh) * page_size + r) * D;
-  };
-  // The loads of tile t.  Keys, as the first operand of the score products: lane (r16, kg) holds, of the four
-  // keys 4 r16 + kt, features 32 s + 8 kg .. + 8.  Values: the lane's chunk of eight features of the value rows
-  // of its NI keys.  Keys beyond pos are read from key pos (they are masked, their probabilities are zero).
-  auto issue = [&](int t, bf16x8_t (*kreg)[KS], uint4* vreg) {
-    const int base = lo + (t << 6);
-    long ko[4], vo[NI];
-#pragma unroll
-    for (int kt = 0; kt < 4; ++kt) {
-      const int u = base + 4 * r16 + kt;
-      ko[kt] = row_off(u <= pos ? u : pos) + kg * 8;
-    }
-#pragma unroll
-    for (int i = 0; i < NI; ++i) {
-      const int uu = base + kq + i * KG;
-      vo[i] = row_off(uu <= pos ? uu : pos) + dc * 8;
-    }
-#pragma unroll
-    for (int kt = 0; kt < 4; ++kt)
-#pragma unroll
-      for (int st = 0; st < KS; ++st) {
-        if (32 * st + 8 * kg < D)
-          kreg[kt][st] = *reinterpret_cast<const bf16x8_t*>(kcache + ko[kt] + 32 * st);
-        else
-          kreg[kt][st] = bf16x8_t{0, 0, 0, 0, 0, 0, 0, 0};
-      }
-#pragma unroll
-    for (int i = 0; i < NI; ++i) vreg[i] = *reinterpret_cast<const uint4*>(vcache + vo[i]);
-  };
-
-  // Loads in the order of what they wait for: the queries, the norm weights and the step's own key and value
-  // (they wait for nothing), the rotation factors and the page numbers (for the position), the key and value rows
-  // (for the page numbers).  Loads return in order, so the queries are normed and rotated while the rows are on
-  // their way.
-  // the queries as the second operand: lane (r16, kg) holds head r16's features 32 s + 8 kg .. + 8
-  // (lanes past the group load head 0's: every lane loads, no branch hides a load from the compiler's count)
-  bf16x8_t qreg[KS];
-#pragma unroll
-  for (int st = 0; st < KS; ++st) {
-    if (32 * st + 8 * kg < D)
-      qreg[st] = *reinterpret_cast<const bf16x8_t*>(q + (size_t)seq * q_stride + (size_t)(kvh * G + (r16 < G ? r16 : 0)) * D + 32 * st + 8 * kg);
-    else
-      qreg[st] = bf16x8_t{0, 0, 0, 0, 0, 0, 0, 0};
-    if (!RAW && r16 >= G) qreg[st] = bf16x8_t{0, 0, 0, 0, 0, 0, 0, 0};
-  }
-  // Every wavefront keeps a copy of its own of the step's key and value in LDS (the wavefront whose tile holds the
-  // new key reads them there: the cache's rows were loaded before they were written), so no wavefront waits for
-  // another; wavefront 0 of the block whose keys end with the new one also writes them to the cache.
-  __shared__ __align__(16) uint16_t knew[RAW ? W : 1][RAW ? D : 8], vnew[RAW ? W : 1][RAW ? D : 8];
-  const bool has_new = RAW && raw.write_kv && t0 < t1 && t1 == tiles;   // this block's keys end with the new one
-  constexpr int E = D >= 64 ? D / 64 : 1;
-  float qw8[RAW ? KS : 1][8], c8[RAW ? KS / 2 : 1][8], s8[RAW ? KS / 2 : 1][8];
-  float kraw_f[E], kw_f[E], kc_f = 1.f, ks_f = 0.f;
-  bf16 vraw_b[E];
-  if constexpr (RAW != 0) {
-    if (raw.qw) {
-#pragma unroll
-      for (int st = 0; st < KS; ++st) load8f(raw.qw + 32 * st + 8 * kg, qw8[st]);
-    }
-    const bf16* kraw = q + (size_t)seq * q_stride + (size_t)(nh + kvh) * D;
-    const bf16* vraw = q + (size_t)seq * q_stride + (size_t)(nh + nkv + kvh) * D;
-#pragma unroll
-    for (int e = 0; e < E; ++e) {
-      kraw_f[e] = to_f32(kraw[lane + 64 * e]);
-      vraw_b[e] = vraw[lane + 64 * e];
-      kw_f[e] = raw.kw ? raw.kw[lane + 64 * e] : 1.f;
-    }
-    // (weights and rotation factors in 16-byte loads: the tables' rows and this lane's offsets are multiples of 8)
-#pragma unroll
-    for (int st = 0; st < KS / 2; ++st) {
-      load8f(raw.cos_t + (size_t)pos * (D / 2) + 32 * st + 8 * kg, c8[st]);
-      load8f(raw.sin_t + (size_t)pos * (D / 2) + 32 * st + 8 * kg, s8[st]);
-    }
-    const int pi = E == 2 ? lane : (lane & 31);          // index of this lane's pair of the key
-    kc_f = raw.cos_t[(size_t)pos * (D / 2) + pi];
-    ks_f = raw.sin_t[(size_t)pos * (D / 2) + pi];
-  }
-  bf16x8_t kn[4][KS];
-  uint4 vn[NI];
-  int t = t0 + wave;
-  // (a wavefront without a tile asks for the block's first one: its address is a valid one, and a load behind a
-  // branch would make the compiler wait for every load in flight where it needs the queries)
-  issue(t < t1 ? t : (t0 < tiles ? t0 : 0), kn, vn);
-
-  if constexpr (RAW != 0) {
-    // head norm and rotation of this lane's part of its query: float32 arithmetic on the product's bfloat16
-    // values, rounded to bfloat16 again, as the separate kernel does.  The halves of a rotation pair (i, i + D/2)
-    // are steps KS/2 apart in the same lane.
-    float qf[KS][8];
-    float ss = 0.f;
-#pragma unroll
-    for (int st = 0; st < KS; ++st)
-#pragma unroll
-      for (int j = 0; j < 8; ++j) {
-        qf[st][j] = (float)qreg[st][j];
-        ss += qf[st][j] * qf[st][j];
-      }
-    if (raw.qw) {
-      const float inv = norm_inverse(group4_sum(ss), (float)D, raw.eps);
-#pragma unroll
-      for (int st = 0; st < KS; ++st)
-#pragma unroll
-        for (int j = 0; j < 8; ++j) qf[st][j] = qf[st][j] * inv * qw8[st][j];
-    }
-#pragma unroll
-    for (int st = 0; st < KS / 2; ++st)
-#pragma unroll
-      for (int j = 0; j < 8; ++j) {
-        const float a = qf[st][j], b = qf[st + KS / 2][j];
-        qf[st][j] = a * c8[st][j] - b * s8[st][j];
-        qf[st + KS / 2][j] = a * s8[st][j] + b * c8[st][j];
-      }
-#pragma unroll
-    for (int st = 0; st < KS; ++st)
-#pragma unroll
-      for (int j = 0; j < 8; ++j) qreg[st][j] = (r16 < G) ? (__bf16)qf[st][j] : (__bf16)0.f;
-    // the new key and value: lane = feature (and feature + 64 for heads of 128)
-    if (raw.write_kv) {
-      float kf[E];
-      float ks = 0.f;
-#pragma unroll
-      for (int e = 0; e < E; ++e) {
-        kf[e] = kraw_f[e];
-        ks += kf[e] * kf[e];
-      }
-      if (raw.kw) {
-        const float inv = norm_inverse(wave_sum_dpp(ks), (float)D, raw.eps);
-#pragma unroll
-        for (int e = 0; e < E; ++e) kf[e] = kf[e] * inv * kw_f[e];
-      }
-      if (E == 2) {
-        const float a = kf[0], b = kf[E - 1];
-        kf[0] = a * kc_f - b * ks_f;
-        kf[E - 1] = a * ks_f + b * kc_f;
-      } else {
-        const float other = __shfl_xor(kf[0], 32, 64);
-        kf[0] = lane < 32 ? kf[0] * kc_f - other * ks_f : other * ks_f + kf[0] * kc_f;
-      }
-      const long row = row_off(pos);
-#pragma unroll
-      for (int e = 0; e < E; ++e) {
-        const bf16 kb = f32_to_bf16(kf[e]);
-        knew[wave][lane + 64 * e] = kb.x;
-        vnew[wave][lane + 64 * e] = vraw_b[e].x;
-        if (has_new && wave == 0) {
-          kcache[row + lane + 64 * e] = kb;
-          vcache[row + lane + 64 * e] = vraw_b[e];
-        }
-      }
-      __builtin_amdgcn_wave_barrier();
-      __builtin_amdgcn_s_waitcnt(0xc07f);  // LDS writes of this wavefront are visible to its own lanes
-    }
-  }
-  const float qscale = scale * DEC_LOG2E;   // scores are scaled after the product, in float32
-
-  // lanes r16 < G keep the running maximum and sum of head r16; every lane keeps its share of all heads' sums
-  float m = -INFINITY, l = 0.f;
-  float acc[G][8];
-#pragma unroll
-  for (int g = 0; g < G; ++g)
-#pragma unroll
-    for (int j = 0; j < 8; ++j) acc[g][j] = 0.f;
-
-  // one tile: scores, online softmax, values
-  auto compute = [&](int t, bf16x8_t (*kc)[KS], uint4* vc) {
-    const int base = lo + (t << 6);
-    if (RAW && has_new && t == tiles - 1) {
-      // the new key's row and the new value's row come from LDS: the cache's rows were loaded before they were written.
-      // So do the places past it, which were loaded from the same row of the cache: their probabilities are zero, but
-      // what that row held before this step (anything: the page may have been another request's) must not meet them
-      const int rel = pos - base;
-#pragma unroll
-      for (int kt = 0; kt < 4; ++kt)
-        if (4 * r16 + kt >= rel) {
-#pragma unroll
-          for (int st = 0; st < KS; ++st) kc[kt][st] = *reinterpret_cast<const bf16x8_t*>(&knew[wave][32 * st + 8 * kg]);
-        }
-#pragma unroll
-      for (int i = 0; i < NI; ++i)
-        if (kq + i * KG >= rel) vc[i] = *reinterpret_cast<const uint4*>(&vnew[wave][dc * 8]);
-    }
-    // sc[kt][i]: head r16, key base + 4 (4 kg + i) + kt
-    f32x4_t sc[4];
-#pragma unroll
-    for (int kt = 0; kt < 4; ++kt) {
-      sc[kt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int st = 0; st < KS; ++st) sc[kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kc[kt][st], qreg[st], sc[kt], 0, 0, 0);
-    }
-    float mx = -INFINITY;
-#pragma unroll
-    for (int kt = 0; kt < 4; ++kt)
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const bool valid = base + 4 * (4 * kg + i) + kt <= pos;
-        float sv = sc[kt][i] * qscale;
-        if (raw.softcap > 0.f) {
-          // cap tanh(x / cap) = cap (1 - 2 / (1 + e^(2 x / cap))), in the base-2 units the scores are held in
-          const float e2 = __builtin_amdgcn_exp2f(sv * (2.f / raw.softcap));
-          sv = raw.softcap * DEC_LOG2E * (1.f - 2.f * __builtin_amdgcn_rcpf(1.f + e2));
-        }
-        sc[kt][i] = valid ? sv : -INFINITY;
-        mx = fmaxf(mx, sc[kt][i]);
-      }
-    const float mn = fmaxf(m, group4_max(mx));   // finite: a tile holds at least one key
-    float sum = 0.f;
-#pragma unroll
-    for (int kt = 0; kt < 4; ++kt)
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        sc[kt][i] = __builtin_amdgcn_exp2f(sc[kt][i] - mn);   // 0 for masked keys
-        sum += sc[kt][i];
-      }
-    const float alpha = __builtin_amdgcn_exp2f(m - mn);
-    l = l * alpha + group4_sum(sum);
-    m = mn;
-    if (r16 < G) {
-#pragma unroll
-      for (int i = 0; i < 4; ++i)
-        *reinterpret_cast<f32x4_t*>(&ps[wave][r16][4 * (4 * kg + i)]) = f32x4_t{sc[0][i], sc[1][i], sc[2][i], sc[3][i]};
-      if (kg == 0) al[wave][r16] = alpha;
-    }
-    __builtin_amdgcn_wave_barrier();
-    __builtin_amdgcn_s_waitcnt(0xc07f);  // LDS writes of this wavefront are visible to its own lanes
-#pragma unroll
-    for (int g = 0; g < G; ++g) {
-      const float a = al[wave][g];
-#pragma unroll
-      for (int j = 0; j < 8; ++j) acc[g][j] *= a;
-    }
-#pragma unroll
-    for (int i = 0; i < NI; ++i) {
-      const uint32_t ww[4] = {vc[i].x, vc[i].y, vc[i].z, vc[i].w};
-      float v[8];
-#pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        v[2 * e] = __uint_as_float(ww[e] << 16);
-        v[2 * e + 1] = __uint_as_float(ww[e] & 0xffff0000u);
-      }
-#pragma unroll
-      for (int g = 0; g < G; ++g) {
-        const float p = ps[wave][g][kq + i * KG];
-#pragma unroll
-        for (int j = 0; j < 8; ++j) acc[g][j] += p * v[j];
-      }
-    }
-    __builtin_amdgcn_wave_barrier();
-  };
-
-  if (PIPE) {
-    // the next tile's loads are in flight while this one is computed: two sets of row registers
-    for (; t < t1; t += W) {
-      bf16x8_t kc[4][KS];
-      uint4 vc[NI];
-#pragma unroll
-      for (int kt = 0; kt < 4; ++kt)
-#pragma unroll
-        for (int st = 0; st < KS; ++st) kc[kt][st] = kn[kt][st];
-#pragma unroll
-      for (int i = 0; i < NI; ++i) vc[i] = vn[i];
-      if (t + W < t1) issue(t + W, kn, vn);
-      compute(t, kc, vc);
-    }
-  } else {
-    // one set of row registers: the first tile's loads were issued above
-    if (t < t1) {
-      compute(t, kn, vn);
-      t += W;
-    }
-    for (; t < t1; t += W) {
-      issue(t, kn, vn);
-      compute(t, kn, vn);
-    }
-  }
-  // key groups of a wavefront hold partial sums over different keys for the same features: add them
-#pragma unroll
-  for (int g = 0; g < G; ++g)
-#pragma unroll
-    for (int j = 0; j < 8; ++j) {
-      float v = acc[g][j];
-      for (int o = DC; o < 64; o <<= 1) v += __shfl_xor(v, o, 64);
-      acc[g][j] = v;
-    }
-  if (kq == 0) {
-#pragma unroll
-    for (int g = 0; g < G; ++g)
-#pragma unroll
-      for (int j = 0; j < 8; ++j) wacc[wave][g][dc * 8 + j] = acc[g][j];
-  }
-  if (lane < G) {
-    wm[wave][lane] = m;
-    wl[wave][lane] = l;
-  }
-  __syncthreads();
-
-  // merge the wavefronts, in wavefront order
-  const size_t unit = ((size_t)seq * nkv + kvh) * nsplit + split;  // this block's partial
-  for (int i = tid; i < G * D; i += blockDim.x) {
-    int g = i / D, j = i - g * D;
-    float M = -INFINITY;
-    for (int w = 0; w < W; ++w) M = fmaxf(M, wm[w][g]);
-    float o = 0.f, L = 0.f;
-    if (M > -INFINITY)
-      for (int w = 0; w < W; ++w)
-        if (wm[w][g] > -INFINITY) {
-          float f = __builtin_amdgcn_exp2f(wm[w][g] - M);
-          o += wacc[w][g][j] * f;
-          L += wl[w][g] * f;
-        }
-    if (nsplit == 1) {
-      // (a sink's score is 0; the maxima are in base-2 units of the scaled scores)
-      if (raw.sink || raw.sinks)
-        L += M > -INFINITY ? __builtin_amdgcn_exp2f((raw.sinks ? raw.sinks[kvh * G + g] * DEC_LOG2E : 0.f) - M) : 1.f;
-      out[out_index(seq, (kvh * G + g) * D + j, nh * D, out_tiles)] = f32_to_bf16(o / L);
-    } else {
-      part_o[(unit * G + g) * D + j] = o;
-      if (j == 0) {
-        part_ml[(unit * G + g) * 2] = M;
-        part_ml[(unit * G + g) * 2 + 1] = L;
-      }
-    }
-  }
-}
 
 // Merge the splits of each (sequence, head), in split order.  One block per (sequence, key head).  The splits'
 // maxima and sums go through LDS, so that each head's weights are computed once and the loads of the partial
 // outputs are independent of one another.
-#define DEC_MAXSPLIT 64
 __global__ void attention_decode_merge_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml,
                                               bf16* __restrict__ out, int nsplit, int nh, int nkv, int G, int D,
                                               int out_tiles, int sink, const float* __restrict__ sinks) {
@@ -495,7 +88,7 @@ static int launch_decode_w(int G, dim3 grid, hipStream_t stream, const bf16* q, 
 #define GS_RUN(GG)                                                                                                     \
   attention_decode_kernel<D, GG, WV, RAW><<<grid, WV * 64, 0, stream>>>(                                 \
       q, q_stride, kc, vc, positions, bt, max_blocks, page_size, page_magic, window, scale, out, part_o, part_ml, nh, \
-      nkv, out_tiles, raw)
+      nkv, out_tiles, raw, DecodeMaps{})
   switch (G) {
     case 1: GS_RUN(1); break;
     case 2: GS_RUN(2); break;
@@ -511,21 +104,13 @@ static int launch_decode_w(int G, dim3 grid, hipStream_t stream, const bf16* q, 
   return 0;
 }
 
-static int g_decode_cus = 0;   // compute units of the device, asked for once
-
 template <int D, int RAW>
 static int launch_decode(int G, dim3 grid, hipStream_t stream, const bf16* q, int q_stride, bf16* kc, bf16* vc,
                          const int* positions, const int* bt, int max_blocks, int page_size, unsigned page_magic,
                          int window, float scale, bf16* out, float* part_o, float* part_ml, int nh, int nkv,
                          int out_tiles, DecodeRaw raw) {
-  if (g_decode_cus == 0) {
-    int dev = 0, n = 0;
-    if (hipGetDevice(&dev) != hipSuccess || hipDeviceGetAttribute(&n, hipDeviceAttributeMultiprocessorCount, dev) != hipSuccess || n <= 0)
-      n = 256;
-    g_decode_cus = n;
-  }
   const long blocks = (long)grid.x * grid.y * grid.z;
-  if (D <= 64 && blocks > 1L * g_decode_cus)
+  if (D <= 64 && blocks > 1L * decode_compute_units())
     return launch_decode_w<D, RAW, 4>(G, grid, stream, q, q_stride, kc, vc, positions, bt, max_blocks, page_size, page_magic,
                                       window, scale, out, part_o, part_ml, nh, nkv, out_tiles, raw);
   return launch_decode_w<D, RAW, DEC_WAVES>(G, grid, stream, q, q_stride, kc, vc, positions, bt, max_blocks, page_size,

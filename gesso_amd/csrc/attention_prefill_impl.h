@@ -22,7 +22,17 @@
 // tile walks those of them that lie before its window's first key in a walk of their own, ahead of the window's.
 // Tiles of queries come
 // from the host: tile i covers rows tile_row[i] .. + tile_n[i] (at most 16 QT) of the flattened tokens, of
-// sequence tile_seq[i].  Exponentials are base 2 on scores scaled by log2(e): one v_exp_f32 each.  q (T, q_stride), head h at [h D, (h+1) D); caches (pages, nkv, page_size, D); out (T, nh D).
+// sequence tile_seq[i].
+//
+// MAPS = 2: attention as the difference of two softmax maps over one value row (attention_maps.hip has the definition).
+// The G wavefronts are then the 2 maps of G / 2 query heads: wavefront w computes map w % 2 of head w / 2, over keys of D
+// features of which the cache holds a head's two side by side, and values DV wide.  A softmax weight enters the value
+// product as two bfloat16 terms (its rounding and the rounding of the remainder), so that the weights keep sixteen bits
+// where the two maps' sums nearly cancel.  At the end the second map's wavefront hands its sums to the first one's, which
+// takes the difference, norms and gates it.  Groups of more heads than a block has wavefronts for are cut into `parts`
+// blocks.
+//
+// Exponentials are base 2 on scores scaled by log2(e): one v_exp_f32 each.  q (T, q_stride), head h at [h D, (h+1) D); caches (pages, nkv, page_size, D); out (T, nh D).
 #pragma once
 #include <type_traits>
 
@@ -40,24 +50,27 @@ typedef __attribute__((ext_vector_type(4))) float f32x4_t;
 // KSPLIT: sets of G wavefronts that share a tile's keys between them, step by step in turn, and add up their
 // (maximum, sum, accumulator) at the end.  A step is a long chain of dependent instructions for one wavefront;
 // the last tiles of a long prompt walk the most keys and set the kernel's time, so their walk is shared out.
-template <int D, int G, int QT, int KSPLIT>
+template <int D, int G, int QT, int KSPLIT, int DV = D, int MAPS = 1>
 __global__ __launch_bounds__(G * KSPLIT * 64) void attention_prefill_kernel(
     const bf16* __restrict__ q, int q_stride, const bf16* __restrict__ kcache, const bf16* __restrict__ vcache,
     const int* __restrict__ positions, const int* __restrict__ tile_seq, const int* __restrict__ tile_row,
     const int* __restrict__ tile_n, const int* __restrict__ block_table, int max_blocks, int page_size,
     unsigned page_magic, int window, float scale, bf16* __restrict__ out, int nh, int nkv, int chunk, int sink,
-    float softcap, int keep_first, const float* __restrict__ sinks) {
-  constexpr int PF_KSTEP = D <= 64 ? 64 : 32;   // keys per step: what three sets of row registers allow
+    float softcap, int keep_first, const float* __restrict__ sinks, MapsEnd me) {
+  static_assert(MAPS == 1 || (MAPS == 2 && G % 2 == 0), "two maps a head, a wavefront each");
+  constexpr int PF_KSTEP = D <= 64 && DV <= 64 ? 64 : 32;   // keys per step: what three sets of row registers allow
   constexpr int KK = D / 32;   // feature steps of the score product
-  constexpr int DT = D / 16;   // feature tiles of the output
+  constexpr int DT = DV / 16;  // feature tiles of the output
   constexpr int NB = PF_KSTEP / 16;   // blocks of 16 keys per step
   constexpr int GT = G * 64;       // threads of a set of wavefronts
-  __shared__ uint16_t vt[KSPLIT][D][PF_KSTEP + PF_PAD];
+  __shared__ uint16_t vt[KSPLIT][DV][PF_KSTEP + PF_PAD];
   __shared__ int pages[PF_MAXPAGES];
   // Blocks in launch order: key head fastest, tiles from the last one back.  Late tiles walk the most keys, so the
   // longest walks all start first whatever their head; and consecutive blocks go to consecutive dies, so a die sees
   // few key heads and their pages stay in its L2.
+  // (nkv: blocks a tile, the key heads times the parts their groups are cut into)
   const int kvh = blockIdx.x % nkv, tile = (int)(gridDim.x / nkv) - 1 - (int)(blockIdx.x / nkv);
+  const int kvc = MAPS == 1 ? kvh : kvh / me.parts, nkc = MAPS == 1 ? nkv : nkv / me.parts;   // the cache's key head, and their number
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int r16 = lane & 15, kg = lane >> 4;
   const int grp = wave / G, gtid = tid - grp * GT;                 // the set, and the thread within it
@@ -115,11 +128,13 @@ __global__ __launch_bounds__(G * KSPLIT * 64) void attention_prefill_kernel(
     if (clamp) u = u < win_first ? win_first : (u > win_last ? win_last : u);
     const int blk = (int)__umulhi((unsigned)u, page_magic);
     const int offs = u - blk * page_size;
-    return (((size_t)pages[blk - win_blk] * nkv + kvh) * page_size + offs) * D;
+    return ((size_t)pages[blk - win_blk] * nkc + kvc) * page_size + offs;
   };
   // The loads of a step are issued two steps ahead and land in registers while the steps before are computed:
   // three sets of row registers, used in turn (the step loop is unrolled by three, so the turns are static).
-  constexpr int VPT = (PF_KSTEP * (D / 8) + GT - 1) / GT;   // value chunks per thread and step
+  constexpr int VC = DV / 8;                                // 16-byte chunks of a value row
+  const int kcol = kg * 8 + (MAPS == 1 ? 0 : wave % MAPS * D);   // this lane's first feature in a cached key row
+  constexpr int VPT = (PF_KSTEP * VC + GT - 1) / GT;   // value chunks per thread and step
   bf16x8_t kb[3][NB][KK];
   uint4 vb[3][VPT];
   // (steps that lie wholly inside the window's keys need no clamping: `inner`, a compile-time flag)
@@ -128,15 +143,15 @@ __global__ __launch_bounds__(G * KSPLIT * 64) void attention_prefill_kernel(
     constexpr bool CLAMP = !decltype(inner)::value;
 #pragma unroll
     for (int b = 0; b < NB; ++b) {
-      const bf16* krow = kcache + row_of(k0 + b * 16 + r16, CLAMP) + kg * 8;   // the key whose row this lane loads
+      const bf16* krow = kcache + row_of(k0 + b * 16 + r16, CLAMP) * (MAPS * D) + kcol;   // the key whose row this lane loads
 #pragma unroll
       for (int kk = 0; kk < KK; ++kk) kb[S][b][kk] = *reinterpret_cast<const bf16x8_t*>(krow + kk * 32);
     }
 #pragma unroll
     for (int x = 0; x < VPT; ++x) {
-      const int i = (gtid + x * GT) % (PF_KSTEP * (D / 8));
-      const int key = i / (D / 8), c = i % (D / 8);
-      vb[S][x] = *reinterpret_cast<const uint4*>(vcache + row_of(k0 + key, CLAMP) + c * 8);
+      const int i = (gtid + x * GT) % (PF_KSTEP * VC);
+      const int key = i / VC, c = i % VC;
+      vb[S][x] = *reinterpret_cast<const uint4*>(vcache + row_of(k0 + key, CLAMP) * DV + c * 8);
     }
   };
   auto fetch = [&](auto stage, int k0) {
@@ -164,8 +179,8 @@ __global__ __launch_bounds__(G * KSPLIT * 64) void attention_prefill_kernel(
 #pragma unroll
     for (int x = 0; x < VPT; ++x) {
       const int i = gtid + x * GT;
-      if (i < PF_KSTEP * (D / 8)) {
-        const int key = i / (D / 8), c = i % (D / 8);
+      if (i < PF_KSTEP * VC) {
+        const int key = i / VC, c = i % VC;
         const uint32_t ww[4] = {vb[S][x].x, vb[S][x].y, vb[S][x].z, vb[S][x].w};
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
@@ -201,7 +216,7 @@ __global__ __launch_bounds__(G * KSPLIT * 64) void attention_prefill_kernel(
           else s[t][b * 4 + i] = sv;
         }
     }
-    bf16x8_t pf[QT][NB / 2];
+    bf16x8_t pf[QT][NB / 2], pl[MAPS > 1 ? QT : 1][MAPS > 1 ? NB / 2 : 1];
 #pragma unroll
     for (int t = 0; t < QT; ++t) {
       float mloc = s[t][0];
@@ -228,6 +243,7 @@ __global__ __launch_bounds__(G * KSPLIT * 64) void attention_prefill_kernel(
         const float pj = none ? 0.f : __builtin_amdgcn_exp2f(fmaf(s[t][j], sc, nm));
         lsum += pj;
         pf[t][j / 8][j % 8] = (__bf16)pj;
+        if constexpr (MAPS > 1) pl[t][j / 8][j % 8] = (__bf16)(pj - (float)pf[t][j / 8][j % 8]);
       }
       l[t] += group4_sum(lsum);
     }
@@ -244,7 +260,10 @@ __global__ __launch_bounds__(G * KSPLIT * 64) void attention_prefill_kernel(
         a.u2[0] = *reinterpret_cast<const uint2*>(&vt[grp][dt * 16 + r16][ns * 32 + kg * 4]);
         a.u2[1] = *reinterpret_cast<const uint2*>(&vt[grp][dt * 16 + r16][ns * 32 + 16 + kg * 4]);
 #pragma unroll
-        for (int t = 0; t < QT; ++t) acc[t][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.v, pf[t][ns], acc[t][dt], 0, 0, 0);
+        for (int t = 0; t < QT; ++t) {
+          acc[t][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.v, pf[t][ns], acc[t][dt], 0, 0, 0);
+          if constexpr (MAPS > 1) acc[t][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.v, pl[t][ns], acc[t][dt], 0, 0, 0);
+        }
       }
   };
   const int last_lo = lo_of(last_key);
@@ -325,7 +344,48 @@ __global__ __launch_bounds__(G * KSPLIT * 64) void attention_prefill_kernel(
         }
       }
     }
-    if (grp > 0) return;
+    if (MAPS == 1 && grp > 0) return;
+  }
+  if constexpr (MAPS == 2) {
+    // the second map's sums go to the first map's wavefront, one tile of queries at a time; lane (query r16, kg) of both
+    // holds the same features of the same query
+    __shared__ float other[G / 2][64][DT * 4 + 1];
+#pragma unroll
+    for (int t = 0; t < QT; ++t) {
+      const float inv = l[t] > 0.f ? 1.0f / l[t] : 0.f;        // (a lane without a query has seen no key)
+      __syncthreads();
+      if (grp == 0 && wave % 2 == 1) {
+#pragma unroll
+        for (int dt = 0; dt < DT; ++dt)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) other[wave / 2][lane][dt * 4 + i] = acc[t][dt][i] * inv;
+      }
+      __syncthreads();
+      if (grp == 0 && wave % 2 == 0) {
+        float ss = 0.f;
+#pragma unroll
+        for (int dt = 0; dt < DT; ++dt)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+            acc[t][dt][i] = acc[t][dt][i] * inv - me.lam * other[wave / 2][lane][dt * 4 + i];
+            ss += acc[t][dt][i] * acc[t][dt][i];
+          }
+        const int row = row0 + (live[t] ? t * 16 + r16 : 0);
+        float f = norm_inverse(group4_sum(ss), (float)DV, me.eps) * me.out_scale;
+        if (me.gate_col >= 0) f *= 1.f / (1.f + expf(-to_f32(q[(size_t)row * q_stride + me.gate_col + h / 2])));
+        bf16* orow = out + (size_t)row * (nh / 2) * DV + (size_t)(h / 2) * DV;
+        if (live[t]) {
+#pragma unroll
+          for (int dt = 0; dt < DT; ++dt) {
+            uint2 o;
+            o.x = (uint32_t)f32_to_bf16(acc[t][dt][0] * f).x | ((uint32_t)f32_to_bf16(acc[t][dt][1] * f).x << 16);
+            o.y = (uint32_t)f32_to_bf16(acc[t][dt][2] * f).x | ((uint32_t)f32_to_bf16(acc[t][dt][3] * f).x << 16);
+            *reinterpret_cast<uint2*>(orow + dt * 16 + kg * 4) = o;
+          }
+        }
+      }
+    }
+    return;
   }
 #pragma unroll
   for (int t = 0; t < QT; ++t) {
@@ -334,7 +394,7 @@ __global__ __launch_bounds__(G * KSPLIT * 64) void attention_prefill_kernel(
     // (a head's own sink has the score sinks[h], unscaled and uncapped)
     if (sink || sinks) l[t] += m[t] == -INFINITY ? 1.f : __builtin_amdgcn_exp2f((sinks ? sinks[h] * PF_LOG2E : 0.f) - m[t]);
     const float inv = 1.0f / l[t];
-    bf16* orow = out + (size_t)(row0 + t * 16 + r16) * nh * D + (size_t)h * D;
+    bf16* orow = out + (size_t)(row0 + t * 16 + r16) * nh * DV + (size_t)h * DV;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) {
       uint2 o;
@@ -355,7 +415,7 @@ static int launch_prefill(int G, dim3 grid, hipStream_t stream, const bf16* q, i
   if constexpr (KSPLIT > 1 && GG > 4) return -1;                                                                        \
   else attention_prefill_kernel<D, GG, QT, KSPLIT><<<grid, GG * KSPLIT * 64, 0, stream>>>(q, q_stride, kc, vc, positions, tile_seq, tile_row, \
                                                                 tile_n, bt, max_blocks, page_size, page_magic, window, \
-                                                                scale, out, nh, nkv, chunk, sink, softcap, keep_first, sinks)
+                                                                scale, out, nh, nkv, chunk, sink, softcap, keep_first, sinks, MapsEnd{})
   switch (G) {
     case 1: GS_RUN(1); break;
     case 2: GS_RUN(2); break;
@@ -386,4 +446,31 @@ static int prefill_for_width(const PrefillCall& c) {
   if (c.tile_rows == 16) return split ? launch_prefill<D, 1, 2>(GS_ARGS) : launch_prefill<D, 1, 1>(GS_ARGS);
   return split ? launch_prefill<D, 2, 2>(GS_ARGS) : launch_prefill<D, 2, 1>(GS_ARGS);
 #undef GS_ARGS
+}
+
+// Two maps a head (MAPS = 2): groups of 1, 2 or 4 query heads a block; c.nh counts the maps of all heads, c.nkv the blocks a
+// tile (key heads times parts).
+template <int D, int DV>
+static int prefill_maps_for_width(const PrefillCall& c, const MapsEnd& me) {
+  dim3 grid((unsigned)c.ntiles * (unsigned)c.nkv);
+  const int G = c.nh / c.nkv;
+#define GS_MAPS(GG, QT, KS)                                                                                                 \
+  attention_prefill_kernel<D, GG, QT, KS, DV, 2><<<grid, GG * KS * 64, 0, c.stream>>>(                                      \
+      c.q, c.q_stride, c.kc, c.vc, c.positions, c.tile_seq, c.tile_row, c.tile_n, c.bt, c.max_blocks, c.page_size,          \
+      c.page_magic, c.window, c.scale, c.out, c.nh, c.nkv, 0, 0, 0.f, 0, nullptr, me)
+#define GS_MAPS_G(QT)                        \
+  switch (G) {                               \
+    case 2: GS_MAPS(2, QT, 2); break;        \
+    case 4: GS_MAPS(4, QT, 2); break;        \
+    case 8: GS_MAPS(8, QT, 1); break;        \
+    default: return -1;                      \
+  }
+  if (c.tile_rows == 16) {
+    GS_MAPS_G(1)
+  } else {
+    GS_MAPS_G(2)
+  }
+#undef GS_MAPS_G
+#undef GS_MAPS
+  return 0;
 }

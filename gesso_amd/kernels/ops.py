@@ -427,6 +427,68 @@ def attention_maps(rows, kcache, vcache, positions, seq_of_token, block_table, p
     return out
 
 
+def attention_prefill_maps_supports(nh: int, nkv: int, d: int, vd: int) -> bool:
+    return bool(lib().gs_attention_prefill_maps_supports(nh, nkv, d, vd))
+
+
+def attention_prefill_maps(rows, kcache, vcache, positions, tiles, block_table, page_size, window, scale, lam: float,
+                           eps: float, out_scale: float, gate_col: int, nh, nkv, d, vd, out: torch.Tensor = None,
+                           tile_rows: int = 16) -> torch.Tensor:
+    """:func:`attention_maps` for prompt portions on the matrix cores (bfloat16).  ``tiles``: int32 ``(3, ntiles)`` as
+    :func:`attention_prefill` takes them."""
+    T = rows.shape[0]
+    _maps_operands(rows, kcache, vcache, positions, block_table, page_size, gate_col, nh, nkv, d, vd, "attention_prefill_maps")
+    _need(rows.dtype == torch.bfloat16, "attention_prefill_maps takes bfloat16")
+    _i32(positions, T, "positions")
+    _need(tiles.dtype == torch.int32 and tiles.dim() == 2 and tiles.shape[0] == 3 and tiles.is_cuda and tiles.is_contiguous(),
+          "tiles must be int32 (3, ntiles)")
+    if out is None:
+        out = torch.empty((T, nh * vd), dtype=rows.dtype, device=rows.device)
+    _need(out.shape == (T, nh * vd) and out.dtype == rows.dtype and out.is_contiguous(), "attention_prefill_maps: out has the wrong shape or type")
+    _check(lib().gs_attention_prefill_maps(_p(rows), rows.shape[1], _p(kcache), _p(vcache), _p(positions), _p(tiles[0]),
+                                           _p(tiles[1]), _p(tiles[2]), tiles.shape[1], _p(block_table), block_table.shape[1],
+                                           page_size, window or 0, scale, lam, eps, out_scale, gate_col, _p(out), nh, nkv, d,
+                                           vd, tile_rows, _stream()))
+    return out
+
+
+def attention_decode_maps_supports(nh: int, nkv: int, d: int, vd: int) -> bool:
+    return bool(lib().gs_attention_decode_maps_supports(nh, nkv, d, vd))
+
+
+def attention_decode_maps_blocks(nh: int, nkv: int) -> int:
+    """How many blocks a sequence makes in :func:`attention_decode_maps` for one split of its keys."""
+    return int(lib().gs_attention_decode_maps_blocks(nh, nkv))
+
+
+_maps_ws = {}
+
+
+def attention_decode_maps(rows, kcache, vcache, positions, block_table, page_size, window, scale, lam: float, eps: float,
+                          out_scale: float, gate_col: int, nh, nkv, d, vd, nseq: int, nsplit: int,
+                          out: torch.Tensor = None) -> torch.Tensor:
+    """:func:`attention_maps` for one query per sequence (bfloat16): sequence ``i`` is row ``i``, its keys split over
+    ``nsplit`` blocks."""
+    _maps_operands(rows, kcache, vcache, positions, block_table, page_size, gate_col, nh, nkv, d, vd, "attention_decode_maps")
+    _need(rows.dtype == torch.bfloat16 and rows.shape[0] >= nseq, "attention_decode_maps takes bfloat16, a row a sequence")
+    _i32(positions, nseq, "positions")
+    _need(block_table.shape[0] >= nseq, "block_table must be int32 (nseq, max_blocks)")
+    ws = None
+    if nsplit > 1:
+        key = (rows.device, nseq, nh, vd, nsplit)
+        ws = _maps_ws.get(key)
+        if ws is None:
+            floats = int(lib().gs_attention_decode_maps_workspace(nseq, nh, vd, nsplit))
+            ws = _maps_ws[key] = torch.empty(max(1, floats), dtype=torch.float32, device=rows.device)
+    if out is None:
+        out = torch.empty((nseq, nh * vd), dtype=rows.dtype, device=rows.device)
+    _need(out.shape == (nseq, nh * vd) and out.dtype == rows.dtype and out.is_contiguous(), "attention_decode_maps: out has the wrong shape or type")
+    _check(lib().gs_attention_decode_maps(_p(rows), rows.shape[1], _p(kcache), _p(vcache), _p(positions), _p(block_table),
+                                          block_table.shape[1], page_size, window or 0, scale, lam, eps, out_scale, gate_col,
+                                          _p(out), _p(ws), nseq, nh, nkv, d, vd, nsplit, _stream()))
+    return out
+
+
 # ---------------------------------------------------------------------- linear attention
 
 _ACTS = {None: 0, "none": 0, "silu": 1}

@@ -71,12 +71,45 @@ class MapAttention(Part):
             o = self.attend(rows, ctx, cache)
         return rt.linear(o, self.w_out)
 
-    def attend(self, rows, ctx, cache) -> torch.Tensor:
-        """The heads' outputs, normed and gated: ``(T, n_heads * value_dim)``."""
+    def _single(self, rows, ctx, cache, nseq: int, out):
+        """The first ``nseq`` sequences, one query each (their rows are the first ``nseq`` rows)."""
         s, ops = self.spec, self.rt.ops
+        longest = ctx.max_kv_len if ctx.max_kv_len is not None else cache.block_table.shape[1] * cache.page_size
+        if s.window:
+            longest = min(longest, s.window)
+        # keys are split over blocks only where the batch alone does not fill the chip, 1,024 keys a split and more
+        blocks = ops.attention_decode_maps_blocks(s.n_heads, s.n_kv_heads)
+        nsplit = max(1, min(-(-longest // 64) // 16, 64, 256 // max(1, nseq * blocks)))
+        return ops.attention_decode_maps(rows, cache.k, cache.v, ctx.positions, cache.block_table, cache.page_size, *self._rule(),
+                                         nseq, nsplit, out=out)
+
+    def _rule(self):
+        """Window, scale, share, norm, gate and sizes, in the order in which the kernels' faces take them."""
+        s = self.spec
+        return (s.window, s.scale, self.lam, s.eps, 1.0 - s.share, self.og if s.head_gate else -1, s.n_heads, s.n_kv_heads,
+                s.map_dim, s.value_dim)
+
+    def attend(self, rows, ctx, cache) -> torch.Tensor:
+        """The heads' outputs, normed and gated: ``(T, n_heads * value_dim)``.  The general kernel takes every size and
+        both precisions; the kernels for prompt portions and for single queries take over where they take the sizes."""
+        s, ops = self.spec, self.rt.ops
+        sizes = (s.n_heads, s.n_kv_heads, s.map_dim, s.value_dim)
+        fast = rows.dtype == torch.bfloat16 and cache.page_size >= 2 and rows.shape[1] % 8 == 0
+        single = fast and ops.attention_decode_maps_supports(*sizes)
+        if single and ctx.all_single:
+            return self._single(rows, ctx, cache, ctx.nseq, None)
+        if fast and not ctx.all_single and ops.attention_prefill_maps_supports(*sizes):
+            # decoded tokens at the batch's head go to the kernel for single queries, portions in tiles of queries
+            out = torch.empty((ctx.T, s.n_heads * s.value_dim), dtype=rows.dtype, device=rows.device)
+            lead = ctx.lead_single if single else 0
+            if lead:
+                self._single(rows, ctx, cache, lead, out[:lead])
+            # tiles of 32 share every key and value fragment between two products (maps of 128 have no registers for them)
+            tile = 32 if ctx.max_q_len >= 64 and s.map_dim <= 64 else 16
+            return ops.attention_prefill_maps(rows, cache.k, cache.v, ctx.positions, ctx.query_tiles(tile, lead),
+                                              cache.block_table, cache.page_size, *self._rule(), out=out, tile_rows=tile)
         return ops.attention_maps(rows, cache.k, cache.v, ctx.positions, ctx.seq_of_token, cache.block_table, cache.page_size,
-                                  s.window, s.scale, self.lam, s.eps, 1.0 - s.share, self.og if s.head_gate else -1,
-                                  s.n_heads, s.n_kv_heads, s.map_dim, s.value_dim)
+                                  *self._rule())
 
 
 register("mixer", "map_attention", MapAttention)

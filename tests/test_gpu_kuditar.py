@@ -15,6 +15,7 @@ import numpy as np
 import pytest
 import torch
 
+import plain_bilolix
 import plain_kuditar as P
 import replay as R
 from tiny import random_ids
@@ -336,7 +337,8 @@ def scan_case(ops, dtype, H, G, n, m, lens, cuts, per_channel, delta, seed=0, sl
             j = h // (H // G)
             if per_channel:
                 alpha = decs[s][:, 3 + h * n:3 + (h + 1) * n].double()
-                heads.append(P.gated_linear(q[:, j], k[:, j], v[:, h], alpha) if not delta else None)
+                heads.append(P.gated_linear(q[:, j], k[:, j], v[:, h], alpha) if not delta
+                             else plain_bilolix.delta_rule(q[:, j], k[:, j], v[:, h], betas[s][:, 2 + h].double(), alpha))
             else:
                 a = decs[s][:, 3 + h].double()
                 b = betas[s][:, 2 + h].double() if delta else None
