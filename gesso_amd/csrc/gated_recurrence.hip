@@ -21,10 +21,12 @@
 //
 // Long portions, segment by segment.  Over a run of tokens the state goes S -> M S + B with an n x n matrix M (what the
 // decays and the delta rule's corrections do to a state, whatever it holds) and B (what the run writes, starting from
-// nothing).  So the segments of a long portion run side by side: the same kernel gives every segment's B (from a state
-// of zeros) and M (from the identity, with every value zero), gated_state_chain walks a sequence's segments in order
-// (S_(s+1) = M_s S_s + B_s, a product of n x n by n x 16 a block and segment) and leaves every segment's first state,
-// and the kernel runs once more from those states for the outputs.  The same arithmetic in another association.
+// nothing).  So the segments of a long portion run side by side: one launch of the same kernel gives every segment's B (from
+// a state of zeros) and M (further blocks, from the identity, with every value zero), gated_state_chain walks a sequence's
+// segments in order (S_(s+1) = M_s S_s + B_s, a product of n x n by n x 16 a block and segment) and leaves every segment's
+// first state, and the kernel runs once more from those states for the outputs.  Without the delta rule M is diagonal, the
+// product of the run's decays: the blocks of B keep it beside their state, and gated_state_chain_diagonal walks the
+// segments elementwise.  The same arithmetic in another association.
 //
 // delta_rule_prep: what the gated delta rule computes between its convolutions and the recurrence, in float32:
 //   q <- q / sqrt(sum q^2 + unit_eps) * q_scale,  k <- k / sqrt(sum k^2 + unit_eps)        per (token, q/k head), in place
@@ -58,7 +60,8 @@ __global__ void __launch_bounds__(256)
 gated_state_scan_kernel(const TI* __restrict__ x, int ld, int oq, int ok, int ov, int rep, float q_scale,
                         const float* __restrict__ decay, int lda, int oa, const float* __restrict__ beta, int ldb,
                         int ob, float* __restrict__ state, const int* __restrict__ q_start,
-                        const int* __restrict__ slots, float* __restrict__ out, int H, int n, int m) {
+                        const int* __restrict__ slots, float* __restrict__ out, int H, int n, int m,
+                        float* __restrict__ seg_m, float* __restrict__ seg_d) {
   constexpr int NMAX = GR_RG * RMAX;
   constexpr int TB = NMAX <= 128 ? 16 : 8;                 // tokens staged at once
   constexpr int PER = (TB * NMAX + 255) / 256;             // values of q (k, decays) a thread stages
@@ -68,17 +71,27 @@ gated_state_scan_kernel(const TI* __restrict__ x, int ld, int oq, int ok, int ov
   __shared__ __attribute__((aligned(16))) float al[VEC ? TB : 1][VEC ? NMAX : 4];
   __shared__ float vs[TB][GR_COLS];
   __shared__ float a1[TB], bs[TB];
-  const int seq = blockIdx.x, h = blockIdx.y, j0 = blockIdx.z * GR_COLS;
+  // What a run of tokens writes and does (seg_m or seg_d given): blocks of `state`'s columns start from zeros; with seg_m
+  // further blocks start from the identity (n columns, every value zero) and leave their columns there; with seg_d (n a
+  // head and run) the first block of `state` also leaves the product of the run's decays.
+  const bool fresh = seg_m || seg_d;
+  const int zv = (m + GR_COLS - 1) / GR_COLS;
+  const bool ident = (int)blockIdx.z >= zv;
+  const int seq = blockIdx.x, h = blockIdx.y, j0 = (ident ? (int)blockIdx.z - zv : (int)blockIdx.z) * GR_COLS;
+  if (ident) m = n;
+  const bool values = !ident;
   const int tid = threadIdx.x, rg = tid & (GR_RG - 1), jl = tid / GR_RG, j = j0 + jl;
   const int t0 = q_start[seq], t1 = q_start[seq + 1];
   if (t1 <= t0) return;
   const int hq = h / rep;
-  float* S = state + (((size_t)slots[seq] * H + h) * n) * m;
-  float s[RMAX];
+  float* S = (ident ? seg_m : state) + (((size_t)slots[seq] * H + h) * n) * m;
+  float s[RMAX], pr[DELTA ? 1 : RMAX];
 #pragma unroll
   for (int r = 0; r < RMAX; ++r) {
     const int i = rg + GR_RG * r;
-    s[r] = (i < n && j < m) ? S[(size_t)i * m + j] : 0.f;
+    if (fresh) s[r] = ident && i == j ? 1.f : 0.f;
+    else s[r] = (i < n && j < m) ? S[(size_t)i * m + j] : 0.f;
+    if (!DELTA) pr[r] = 1.f;
   }
   // a batch's values on their way: asked for one batch ahead, kept in registers until the batch before has been read
   float rq[PER], rk[PER], ra[VEC ? PER : 1], rv[PERV], r1 = 0.f, rb = 0.f;
@@ -98,7 +111,7 @@ gated_state_scan_kernel(const TI* __restrict__ x, int ld, int oq, int ok, int ov
     for (int u = 0; u < PERV; ++u) {
       const int idx = tid + u * 256;
       const int tt = idx / GR_COLS, c = idx - tt * GR_COLS;
-      rv[u] = (ov >= 0 && idx < nb * GR_COLS && j0 + c < m) ? to_f32(x[(size_t)(tb + tt) * ld + ov + h * m + j0 + c]) : 0.f;
+      rv[u] = (values && idx < nb * GR_COLS && j0 + c < m) ? to_f32(x[(size_t)(tb + tt) * ld + ov + h * m + j0 + c]) : 0.f;
     }
     if (tid < nb) {
       if (!VEC) r1 = decay[(size_t)(tb + tid) * lda + oa + h];
@@ -158,6 +171,7 @@ gated_state_scan_kernel(const TI* __restrict__ x, int ld, int oq, int ok, int ov
 #pragma unroll
     for (int r = 0; r < RMAX; ++r) {
       s[r] *= VEC ? t.a[r] : t.a1;
+      if (!DELTA && seg_d) pr[r] *= VEC ? t.a[r] : t.a1;
       if (DELTA) {
         const float w = s[r] * t.k[r];
         if ((r & 3) == 0) p0 += w; else if ((r & 3) == 1) p1 += w; else if ((r & 3) == 2) p2 += w; else p3 += w;
@@ -198,29 +212,33 @@ gated_state_scan_kernel(const TI* __restrict__ x, int ld, int oq, int ok, int ov
   for (int r = 0; r < RMAX; ++r) {
     const int i = rg + GR_RG * r;
     if (i < n && j < m) S[(size_t)i * m + j] = s[r];
+    if (!DELTA && seg_d && blockIdx.z == 0 && jl == 0 && i < n) seg_d[((size_t)slots[seq] * H + h) * n + i] = pr[r];
   }
 }
 
 extern "C" int gs_gated_state_scan(const void* x, int dtype, int ld, int oq, int ok, int ov, int qk_heads, float q_scale,
                                    const float* decay, int lda, int oa, int per_channel, const float* beta, int ldb,
                                    int ob, float* state, const int* q_start, const int* slots, float* out, int nseq,
-                                   int H, int n, int m, hipStream_t stream) {
+                                   int H, int n, int m, float* seg_m, float* seg_d, hipStream_t stream) {
   GS_REQUIRE(nseq >= 0 && H > 0 && n > 0 && m > 0, "gated_state_scan: bad sizes nseq=%d H=%d n=%d m=%d", nseq, H, n, m);
   GS_REQUIRE(n <= 256, "gated_state_scan: keys of %d features, the kernel holds up to 256", n);
   GS_REQUIRE(qk_heads > 0 && H % qk_heads == 0, "gated_state_scan: %d heads do not share %d queries and keys evenly", H,
              qk_heads);
-  GS_REQUIRE(H <= 65535 && (m + GR_COLS - 1) / GR_COLS <= 65535, "gated_state_scan: too many heads or value columns");
-  // (ov < 0: every value is zero, what the state does to itself over the tokens; out null: the states alone are wanted)
-  GS_REQUIRE(oq >= 0 && ok >= 0 && oq + qk_heads * n <= ld && ok + qk_heads * n <= ld && (ov < 0 || ov + H * m <= ld),
+  GS_REQUIRE(H <= 65535 && m <= 1000000, "gated_state_scan: too many heads or value columns");
+  // (out null: the states alone are wanted)
+  GS_REQUIRE(!((seg_m || seg_d) && out) && !(seg_m && seg_d) && !(seg_d && beta),
+             "gated_state_scan: what a run does to a state is a matrix with the delta rule or a diagonal without, and comes without outputs");
+  GS_REQUIRE(oq >= 0 && ok >= 0 && ov >= 0 && oq + qk_heads * n <= ld && ok + qk_heads * n <= ld && ov + H * m <= ld,
              "gated_state_scan: q, k or v lie outside the rows of %d", ld);
   GS_REQUIRE(decay && oa >= 0 && oa + (per_channel ? H * n : H) <= lda, "gated_state_scan: the decays lie outside their rows of %d", lda);
   GS_REQUIRE(!beta || (ob >= 0 && ob + H <= ldb), "gated_state_scan: the write strengths lie outside their rows of %d", ldb);
   if (nseq == 0) return 0;
-  dim3 grid(nseq, H, (m + GR_COLS - 1) / GR_COLS);
+  dim3 grid(nseq, H, (m + GR_COLS - 1) / GR_COLS + (seg_m ? (n + GR_COLS - 1) / GR_COLS : 0));
+  GS_REQUIRE(grid.z <= 65535, "gated_state_scan: too many value columns");
   const int rep = H / qk_heads;
 #define GR_RUN(TI, R, V, D)                                                                                         \
   gated_state_scan_kernel<TI, R, V, D><<<grid, 256, 0, stream>>>((const TI*)x, ld, oq, ok, ov, rep, q_scale, decay, \
-                                                                 lda, oa, beta, ldb, ob, state, q_start, slots, out, H, n, m)
+                                                                 lda, oa, beta, ldb, ob, state, q_start, slots, out, H, n, m, seg_m, seg_d)
 #define GR_RUN_R(TI, V, D)                   \
   if (n <= 32) GR_RUN(TI, 2, V, D);          \
   else if (n <= 64) GR_RUN(TI, 4, V, D);     \
@@ -353,6 +371,46 @@ extern "C" int gs_gated_state_chain(const float* M, const float* B, float* first
   const size_t lds = (2 * (size_t)n * GR_COLS + (size_t)R * n) * sizeof(float);
   gated_state_chain_kernel<<<grid, 256, lds, stream>>>(M, B, first, state, seq_seg, slots, H, n, m, R);
   GS_LAUNCH_CHECK("gated_state_chain");
+  return 0;
+}
+
+// The same where M is diagonal: d (segments, H, n).  A thread per state element of a sequence walks its segments.
+__global__ void __launch_bounds__(256)
+gated_state_chain_diagonal_kernel(const float* __restrict__ d, const float* __restrict__ B, float* __restrict__ first,
+                                  float* __restrict__ state, const int* __restrict__ seq_seg, const int* __restrict__ slots,
+                                  int H, int n, int m) {
+  const int seq = blockIdx.x, per = H * n * m, e = blockIdx.y * 256 + threadIdx.x;
+  if (e >= per) return;
+  const int s0 = seq_seg[seq], s1 = seq_seg[seq + 1], row = e / m;
+  if (s1 <= s0) return;
+  float* own = state + (size_t)slots[seq] * per + e;
+  float S = *own;
+  for (int sg = s0; sg < s1; sg += 4) {            // (four segments' loads in flight)
+    float dv[4], bv[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const int g = sg + u < s1 ? sg + u : s1 - 1;
+      dv[u] = d[(size_t)g * H * n + row];
+      bv[u] = B[(size_t)g * per + e];
+    }
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      if (sg + u < s1) {
+        first[(size_t)(sg + u) * per + e] = S;
+        S = fmaf(dv[u], S, bv[u]);
+      }
+    }
+  }
+  *own = S;
+}
+
+extern "C" int gs_gated_state_chain_diagonal(const float* d, const float* B, float* first, float* state, const int* seq_seg,
+                                             const int* slots, int nseq, int H, int n, int m, hipStream_t stream) {
+  GS_REQUIRE(nseq >= 0 && H > 0 && n > 0 && m > 0 && (long)H * n * m <= 65535L * 256, "gated_state_chain_diagonal: bad sizes nseq=%d H=%d n=%d m=%d", nseq, H, n, m);
+  if (nseq == 0) return 0;
+  dim3 grid(nseq, gs_ceil_div((long)H * n * m, 256));
+  gated_state_chain_diagonal_kernel<<<grid, 256, 0, stream>>>(d, B, first, state, seq_seg, slots, H, n, m);
+  GS_LAUNCH_CHECK("gated_state_chain_diagonal");
   return 0;
 }
 
