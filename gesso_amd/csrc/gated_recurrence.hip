@@ -274,7 +274,7 @@ __global__ void __launch_bounds__(256)
 gated_state_chain_kernel(const float* __restrict__ M, const float* __restrict__ B, float* __restrict__ first,
                          float* __restrict__ state, const int* __restrict__ seq_seg, const int* __restrict__ slots, int H,
                          int n, int m, int R) {
-  extern __shared__ float ch_s[];             // S and its successor, n x 16 each; then a tile of M, R x n
+  extern __shared__ __attribute__((aligned(16))) float ch_s[];   // S and its successor, n x 16 each; then a tile of M, R x n
   float* S = ch_s;
   float* N = ch_s + (size_t)n * GR_COLS;
   float* Mt = ch_s + 2 * (size_t)n * GR_COLS;
@@ -330,22 +330,41 @@ gated_state_chain_kernel(const float* __restrict__ M, const float* __restrict__ 
       for (int i = rl; i < n; i += 16)
         if (j < m) Fs[(size_t)i * m + j] = S[i * GR_COLS + jl];
     }
+    // a thread's four rows together: a value of S is read once for the four, a row four values at a time where rows allow
+    const float* row[4];
+    float acc[4][4];
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      const int ir = rl + 16 * r, i = r0 + ir;
-      if (ir < R && i < n) {
-        const float* row = Mt + (size_t)ir * n;
-        float a0 = bv[r], a1 = 0.f, a2 = 0.f, a3 = 0.f;
-        int k = 0;
-        for (; k + 3 < n; k += 4) {
-          a0 = fmaf(row[k], S[k * GR_COLS + jl], a0);
-          a1 = fmaf(row[k + 1], S[(k + 1) * GR_COLS + jl], a1);
-          a2 = fmaf(row[k + 2], S[(k + 2) * GR_COLS + jl], a2);
-          a3 = fmaf(row[k + 3], S[(k + 3) * GR_COLS + jl], a3);
+      const int ir = rl + 16 * r;
+      row[r] = Mt + (size_t)(ir < R && r0 + ir < n ? ir : 0) * n;
+      acc[r][0] = bv[r];
+      acc[r][1] = acc[r][2] = acc[r][3] = 0.f;
+    }
+    int k = 0;
+    if (vec) {
+#pragma unroll 2
+      for (; k < n; k += 4) {
+        const float s0v = S[k * GR_COLS + jl], s1v = S[(k + 1) * GR_COLS + jl], s2v = S[(k + 2) * GR_COLS + jl],
+                    s3v = S[(k + 3) * GR_COLS + jl];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const float4 v = *reinterpret_cast<const float4*>(row[r] + k);
+          acc[r][0] = fmaf(v.x, s0v, acc[r][0]);
+          acc[r][1] = fmaf(v.y, s1v, acc[r][1]);
+          acc[r][2] = fmaf(v.z, s2v, acc[r][2]);
+          acc[r][3] = fmaf(v.w, s3v, acc[r][3]);
         }
-        for (; k < n; ++k) a0 = fmaf(row[k], S[k * GR_COLS + jl], a0);
-        N[i * GR_COLS + jl] = (a0 + a1) + (a2 + a3);
       }
+    }
+    for (; k < n; ++k) {
+      const float sv = S[k * GR_COLS + jl];
+#pragma unroll
+      for (int r = 0; r < 4; ++r) acc[r][0] = fmaf(row[r][k], sv, acc[r][0]);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int ir = rl + 16 * r;
+      if (ir < R && r0 + ir < n) N[(r0 + ir) * GR_COLS + jl] = (acc[r][0] + acc[r][1]) + (acc[r][2] + acc[r][3]);
     }
     if (r0 + R >= n) {                         // the segment's last tile: its successor is whole
       __syncthreads();
