@@ -11,6 +11,7 @@ from .models import fazezen as _fazezen  # noqa: F401  registers the architectur
 from .models import togalorn as _togalorn  # noqa: F401  registers the architecture
 from .models import kuditar as _kuditar  # noqa: F401  registers the architecture
 from .models import bilolix as _bilolix  # noqa: F401  registers the architecture
+from .models import vakesun as _vakesun  # noqa: F401  registers the architecture
 from .errors import (ConfigError, GessoError, InvalidPlan, KernelError, NumericalInstability, OutOfPages,
                      OutOfSlots, ResourceLimit, StepFailed, WeightError)
 

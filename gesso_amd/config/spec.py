@@ -53,6 +53,15 @@ class GroupRMSNormSpec:
 
 
 @dataclass(frozen=True)
+class DynTanhSpec:
+    """``tanh(alpha x) w + b``, ``alpha`` one stored number, ``w`` and ``b`` vectors: a norm that computes no statistics of
+    the row."""
+
+    size: int
+    kind: str = "dyn_tanh"
+
+
+@dataclass(frozen=True)
 class RopeSpec:
     """Rotary encoding over the first ``rotary_dim`` features of a head; ``layout``: pairs ``(i, i + rotary_dim/2)``
     (``"half"``) or ``(2i, 2i + 1)`` (``"interleaved"``)."""
@@ -153,7 +162,9 @@ class LatentAttentionSpec:
     order) and ``value_dim`` value features.  ``gated``: head ``h``'s output is multiplied by
     ``sigmoid(W_g x)[h]``; with ``gate_each`` every output feature has a gate of its own (``W_g`` has
     ``n_heads * value_dim`` rows).  ``position`` is the encoding of the ``rot_dim`` part (its ``head_dim`` = ``rot_dim``);
-    its pairs may be laid out either way."""
+    its pairs may be laid out either way.  ``sinks``: the softmax's denominator has one more term ``exp(s_h)``, ``s_h`` a
+    stored number a head.  ``own_rows = False``: the mixer makes no latent rows, it attends over those that an earlier
+    call of the schedule cached (its :class:`LayerCall` names that call) with everything else its own."""
 
     hidden: int
     n_heads: int
@@ -169,6 +180,8 @@ class LatentAttentionSpec:
     gated: bool = True
     kind: str = "latent_attention"
     gate_each: bool = False
+    sinks: bool = False
+    own_rows: bool = True
 
 
 @dataclass(frozen=True)
@@ -267,6 +280,24 @@ class GatedLinearSpec:
 
 
 @dataclass(frozen=True)
+class MatrixMemorySpec:
+    """A matrix memory a head with exponential gates.  ``q`` (times ``key_dim^-0.5``), ``k`` (``n_heads`` heads of ``key_dim``)
+    and ``v`` (of ``value_dim``) are products of the input; ``i = gate_cap tanh((W_i x + b_i) / gate_cap)`` and
+    ``f = log sigmoid(gate_cap tanh((W_f x + b_f) / gate_cap))`` per head.  With a running maximum ``p`` (0 at a request's
+    start), ``p_t = max(f + p_(t-1), i)``: ``S_t = exp(f + p_(t-1) - p_t) S_(t-1) + exp(i - p_t) k v^T`` and ``n_t`` likewise
+    with ``k`` alone, ``o = S^T q / (max(|n . q|, exp(-p)) + 1e-6)``; each head's ``o`` is divided by its root mean square,
+    all heads are multiplied by a weight and by ``sigmoid(W_g x)``, then projected."""
+
+    hidden: int
+    n_heads: int
+    key_dim: int
+    value_dim: int
+    gate_cap: float
+    eps: float
+    kind: str = "matrix_memory"
+
+
+@dataclass(frozen=True)
 class MixerPairSpec:
     """Two mixers side by side that read the same input: ``left_scale * left(x) + right_scale * right(x)``.  Each keeps
     its own cache.  ``branch_norm_eps``: each side's output is first RMS-normed over the model width with a weight of
@@ -298,8 +329,8 @@ class SwiGLUSpec:
 
 @dataclass(frozen=True)
 class MLPSpec:
-    """``W_down act(W_up x)``, no gate and no biases; ``activation``: ``"gelu"`` (the error-function form), ``"gelu_tanh"`` or
-    ``"silu"``."""
+    """``W_down act(W_up x)``, no gate and no biases; ``activation``: ``"gelu"`` (the error-function form), ``"gelu_tanh"``,
+    ``"silu"`` or ``"relu_squared"``."""
 
     hidden: int
     intermediate: int
@@ -428,6 +459,40 @@ class OutNormBlockSpec:
     mult: float = 1.0
     names: Mapping[str, str] = field(compare=False, hash=False, default_factory=dict)
     kind: str = "outnorm"
+
+
+@dataclass(frozen=True)
+class TokenSideSpec:
+    """What a token brings to one layer by itself: with ``e`` the columns ``[offset, offset + dim)`` of its row in a table of
+    ``columns``, ``y = W_proj (gelu_tanh(W_gate h) * e)``, RMS-normed with a weight.  The table may be shared by the layers,
+    each with columns of its own."""
+
+    hidden: int
+    vocab: int
+    dim: int
+    columns: int
+    offset: int
+    eps: float
+    kind: str = "token_side"
+
+
+@dataclass(frozen=True)
+class SandwichBlockSpec:
+    """One block with a norm on both sides of every sub-layer: ``h += mult * norm_b(mixer(norm_a(h)))``, then
+    ``h += mult * norm_d(ffn(norm_c(h)))``, then, with ``side``, ``h += mult * side(h)`` (:class:`TokenSideSpec`).  ``names``
+    as in :class:`BlockSpec` (roles ``mixer_norm.``, ``mixer.``, ``mixer_out_norm.``, ``ffn_norm.``, ``ffn.``,
+    ``ffn_out_norm.``, ``side.``)."""
+
+    mixer: Any
+    mixer_norm: Any
+    mixer_out_norm: Any
+    ffn: Any                           # None = no feed-forward in this block
+    ffn_norm: Any
+    ffn_out_norm: Any
+    side: Any = None
+    mult: float = 1.0
+    names: Mapping[str, str] = field(compare=False, hash=False, default_factory=dict)
+    kind: str = "sandwich"
 
 
 @dataclass(frozen=True)

@@ -117,11 +117,11 @@ static int launch_decode(int G, dim3 grid, hipStream_t stream, const bf16* q, in
                                             page_magic, window, scale, out, part_o, part_ml, nh, nkv, out_tiles, raw);
 }
 
-// Whether this kernel takes the sizes: head widths 16, 32, 64, 128 and groups of up to 8 heads.
+// Whether this kernel takes the sizes: head widths 16, 32, 64, 96, 128 and groups of up to 8 heads.
 extern "C" int gs_attention_decode_supports(int nh, int nkv, int d) {
   if (nkv <= 0 || nh % nkv) return 0;
   int g = nh / nkv;
-  return (d == 16 || d == 32 || d == 64 || d == 128) && g >= 1 && g <= DEC_MAXG;
+  return (d == 16 || d == 32 || d == 64 || d == 96 || d == 128) && g >= 1 && g <= DEC_MAXG;
 }
 
 // Floats of workspace for nseq sequences: partial outputs, then (max, sum) pairs.
@@ -181,6 +181,7 @@ static int decode_entry(const void* q, int q_stride, void* kcache, void* vcache,
       case 16: rc = launch_decode<16, 0>(GS_ARGS, none); break;
       case 32: rc = launch_decode<32, 0>(GS_ARGS, none); break;
       case 64: rc = launch_decode<64, 0>(GS_ARGS, none); break;
+      case 96: rc = launch_decode<96, 0>(GS_ARGS, none); break;
       case 128: rc = launch_decode<128, 0>(GS_ARGS, none); break;
     }
   }

@@ -78,10 +78,11 @@ __global__ __launch_bounds__(W * 64) void attention_decode_kernel(
   static_assert(MAPS == 1 ? DV == D : (MAPS == 2 && !RAW && G % 2 == 0), "values of another width and two maps go together");
   static_assert(!RAW || D == 64 || D == 128, "the fused head norm and rotation are written for heads of 64 and 128");
   constexpr int DC = DV / 8;              // 16-byte chunks per value row
-  constexpr int KG = 64 / DC;             // key groups per wavefront in the value phase
+  constexpr int DL = DC <= 2 ? 2 : DC <= 4 ? 4 : DC <= 8 ? 8 : DC <= 16 ? 16 : DC <= 32 ? 32 : 64;   // lanes a value row: a power of two (those beyond DC idle)
+  constexpr int KG = 64 / DL;             // key groups per wavefront in the value phase
   constexpr int NI = 64 / KG;             // keys per lane in the value phase
   constexpr int KS = (D + 31) / 32;       // steps of 32 features in the score products
-  static_assert(D % 8 == 0 && DV % 8 == 0 && 64 % DC == 0 && G <= 16, "head width must be 8, 16, 32, 64, 128, 256 or 512");
+  static_assert(D % 8 == 0 && DV % 8 == 0 && DC >= 2 && DC <= 64 && G <= 16, "head widths are multiples of 8 from 16 to 512");
   // What the registers allow (256 a lane at eight wavefronts a block): the next tile's rows in flight while
   // this one is computed, for rows of up to 64.
   constexpr bool PIPE = D <= 64 && DV <= 64;
@@ -107,7 +108,9 @@ __global__ __launch_bounds__(W * 64) void attention_decode_kernel(
   const int tper = (tiles + nsplit - 1) / nsplit;
   const int t0 = split * tper, t1 = (t0 + tper < tiles) ? t0 + tper : tiles;
   const int* bt = block_table + (size_t)seq * max_blocks;
-  const int dc = lane % DC, kq = lane / DC;
+  const int kq = lane / DL;
+  const bool dlive = DL == DC || lane % DL < DC;       // (a spare lane loads and sums what its neighbours do, and stores nothing)
+  const int dc = dlive ? lane % DL : DC - 1;
 
   // which row of the caches is key u's (u <= pos)
   // (u / page_size as one multiplication, page_magic = floor(2^32 / page_size) + 1, exact while u page_size < 2^32:
@@ -401,10 +404,10 @@ __global__ __launch_bounds__(W * 64) void attention_decode_kernel(
 #pragma unroll
     for (int j = 0; j < 8; ++j) {
       float v = acc[g][j];
-      for (int o = DC; o < 64; o <<= 1) v += __shfl_xor(v, o, 64);
+      for (int o = DL; o < 64; o <<= 1) v += __shfl_xor(v, o, 64);
       acc[g][j] = v;
     }
-  if (kq == 0) {
+  if (kq == 0 && dlive) {
 #pragma unroll
     for (int g = 0; g < G; ++g)
 #pragma unroll

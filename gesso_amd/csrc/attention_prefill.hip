@@ -3,11 +3,11 @@
 #include "attention_prefill_decl.h"
 
 
-// Head widths 32, 64, 128; groups of 1 to 8 heads (the block has one wavefront per head of the group).
+// Head widths 32, 64, 96, 128; groups of 1 to 8 heads (the block has one wavefront per head of the group).
 extern "C" int gs_attention_prefill_supports(int nh, int nkv, int d) {
   if (nkv <= 0 || nh % nkv) return 0;
   int g = nh / nkv;
-  return (d == 32 || d == 64 || d == 128) && g >= 1 && g <= 8;
+  return (d == 32 || d == 64 || d == 96 || d == 128) && g >= 1 && g <= 8;
 }
 
 extern "C" int gs_attention_prefill(const void* q, int q_stride, const void* kcache, const void* vcache,
@@ -38,6 +38,7 @@ extern "C" int gs_attention_prefill(const void* q, int q_stride, const void* kca
   switch (d) {
     case 32: rc = gs_attention_prefill_d32(c); break;
     case 64: rc = gs_attention_prefill_d64(c); break;
+    case 96: rc = gs_attention_prefill_d96(c); break;
     case 128: rc = gs_attention_prefill_d128(c); break;
   }
   GS_REQUIRE(rc == 0, "attention_prefill: no kernel for this group size");

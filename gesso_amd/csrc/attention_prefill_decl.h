@@ -24,6 +24,7 @@ struct MapsEnd {
 
 int gs_attention_prefill_d32(const PrefillCall& c);
 int gs_attention_prefill_d64(const PrefillCall& c);
+int gs_attention_prefill_d96(const PrefillCall& c);
 int gs_attention_prefill_d128(const PrefillCall& c);
 int gs_attention_prefill_maps_narrow(const PrefillCall& c, const MapsEnd& me, int d, int dv);
 int gs_attention_prefill_maps_wide(const PrefillCall& c, const MapsEnd& me, int d, int dv);

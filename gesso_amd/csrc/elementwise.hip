@@ -19,7 +19,7 @@ void gs_set_error(const char* fmt, ...) {
 
 extern "C" const char* gs_last_error() { return g_err; }
 
-extern "C" int gs_abi_version() { return 13; }
+extern "C" int gs_abi_version() { return 14; }
 
 // ------------------------------------------------------------------ embedding
 
@@ -736,10 +736,15 @@ extern "C" int gs_add_rmsnorm_pair(float* res, const void* d1, const void* d2, i
 
 // in (T, 2F) = gate | up (a product's float32 sums or rounded rows), bias (2F) float32 or absent:
 //   out[t, j] = act(gate[t, j] + bias[j]) * (up[t, j] + bias[F + j])
-// act 0: silu, z / (1 + exp(-z)); act 1: the tanh form of gelu, 0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))).
+// act 0: silu, z / (1 + exp(-z)); act 1: the tanh form of gelu, 0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))); act 2: gelu's
+// error-function form; act 3: the square of relu.
 __device__ __forceinline__ float gated_act(float z, int act) {
   if (act == 0) return z / (1.0f + expf(-z));
   if (act == 2) return 0.5f * z * (1.0f + erff(z * 0.7071067811865476f));
+  if (act == 3) {
+    const float u = z < 0.f ? 0.f : z;               // (NaN stays NaN)
+    return u * u;
+  }
   const float u = 0.7978845608028654f * (z + 0.044715f * z * z * z);
   return 0.5f * z * (1.0f + tanhf(u));
 }
@@ -789,7 +794,7 @@ __global__ void gated_act8_kernel(const TI* __restrict__ in, const float* __rest
 extern "C" int gs_gated_act(const void* in, int in_dtype, const float* bias, void* out, int out_dtype, int T, int F,
                             int act, hipStream_t stream) {
   GS_REQUIRE(T >= 0 && F > 0, "gated_act: bad sizes T=%d F=%d", T, F);
-  GS_REQUIRE(act >= 0 && act <= 2, "gated_act: unknown activation %d", act);
+  GS_REQUIRE(act >= 0 && act <= 3, "gated_act: unknown activation %d", act);
   const long n = (long)T * F;
   if (n == 0) return 0;
   const bool v8 = F % 8 == 0 && ((uintptr_t)in & 15) == 0 && ((uintptr_t)out & 15) == 0 && ((uintptr_t)bias & 15) == 0;
@@ -814,7 +819,7 @@ extern "C" int gs_gated_act(const void* in, int in_dtype, const float* bias, voi
 
 // ------------------------------------------------------------------ an activation alone
 
-// out[i] = act(in[i]): act 0 silu, 1 gelu (tanh form), 2 gelu (error-function form); float32 arithmetic.  VEC: eight values
+// out[i] = act(in[i]): act 0 silu, 1 gelu (tanh form), 2 gelu (error-function form), 3 the square of relu; float32 arithmetic.  VEC: eight values
 // a thread with 16-byte accesses.
 template <typename TI, typename TO, bool VEC>
 __global__ void activate_kernel(const TI* __restrict__ in, TO* __restrict__ out, long n, int act) {
@@ -833,7 +838,7 @@ __global__ void activate_kernel(const TI* __restrict__ in, TO* __restrict__ out,
 
 extern "C" int gs_activate(const void* in, int in_dtype, void* out, int out_dtype, long n, int act, hipStream_t stream) {
   GS_REQUIRE(n >= 0, "activate: bad size");
-  GS_REQUIRE(act >= 0 && act <= 2, "activate: unknown activation %d", act);
+  GS_REQUIRE(act >= 0 && act <= 3, "activate: unknown activation %d", act);
   if (n == 0) return 0;
   const bool v8 = n % 8 == 0 && ((uintptr_t)in & 15) == 0 && ((uintptr_t)out & 15) == 0;
   const int blocks = gs_ceil_div(v8 ? n / 8 : n, 256);

@@ -4,13 +4,16 @@
 //
 //   S <- diag(a_t) S                      a_t: one number per (token, head), or one per (token, head, key channel)
 //   u_t = beta_t (v_t - S^T k_t)          with `delta` (the delta rule: what the state already answers to k_t is taken
-//                                         off the value before it is written);  u_t = v_t without
+//                                         off the value before it is written);  u_t = v_t without, or beta_t v_t where
+//                                         the token has a write strength and no delta rule
 //   S <- S + k_t u_t^T,   o_t = S^T (q_scale q_t)
 //
 // q_t, k_t (n values) and v_t (m values) are columns of a row buffer x (T, ld), float32 or bfloat16: q of head h at
 // [oq + (h / rep) n, ...), k at [ok + (h / rep) n, ...) (rep = H / qk_heads heads share one q and k), v at [ov + h m, ...).
 // The decays are float32 rows (T, lda): a_t of head h at [oa + h] or, per channel, at [oa + h n, ...); beta_t float32 at
-// [ob + h] of rows (T, ldb).  Nothing is rounded below float32 between the rows and the output (T, H m).
+// [ob + h] of rows (T, ldb).  With `ones` a head's last value column is not stored: every value in it is one (the state's
+// column is then the sum of the keys as written and faded), and v of head h has m - 1 columns at [ov + h (m - 1), ...).
+// Nothing is rounded below float32 between the rows and the output (T, H m).
 //
 // gated_state_scan: one block per (sequence, head, tile of 16 value columns).  Thread (rg, jl) = (tid & 15, tid >> 4)
 // holds the state's rows rg, rg + 16, ... of column jl in registers; the sixteen partial sums of a column (S^T k, S^T q)
@@ -55,13 +58,15 @@ __device__ __forceinline__ float gr_sum16(float x) {
 // RMAX: state rows a thread (keys up to 16 RMAX wide).  A thread's rows i = rg + 16 r lie side by side in LDS (place
 // rg RMAX + r), so that it reads them up to sixteen bytes at a time; the places of rows beyond n hold zeros.  The tokens of the next batch are asked for before this
 // batch is computed and land in registers meanwhile.
-template <typename TI, int RMAX, bool VEC, bool DELTA>
+// RULE: 0 values as they are, 1 the delta rule, 2 values times their write strength.
+template <typename TI, int RMAX, bool VEC, int RULE>
 __global__ void __launch_bounds__(256)
 gated_state_scan_kernel(const TI* __restrict__ x, int ld, int oq, int ok, int ov, int rep, float q_scale,
                         const float* __restrict__ decay, int lda, int oa, const float* __restrict__ beta, int ldb,
                         int ob, float* __restrict__ state, const int* __restrict__ q_start,
                         const int* __restrict__ slots, float* __restrict__ out, int H, int n, int m,
-                        float* __restrict__ seg_m, float* __restrict__ seg_d) {
+                        float* __restrict__ seg_m, float* __restrict__ seg_d, int ones) {
+  constexpr bool DELTA = RULE == 1, STRENGTH = RULE != 0;
   constexpr int NMAX = GR_RG * RMAX;
   constexpr int TB = NMAX <= 128 ? 16 : 8;                 // tokens staged at once
   constexpr int PER = (TB * NMAX + 255) / 256;             // values of q (k, decays) a thread stages
@@ -77,6 +82,7 @@ gated_state_scan_kernel(const TI* __restrict__ x, int ld, int oq, int ok, int ov
   const bool fresh = seg_m || seg_d;
   const int zv = (m + GR_COLS - 1) / GR_COLS;
   const bool ident = (int)blockIdx.z >= zv;
+  const int mv = m - ones;                                 // value columns that are stored
   const int seq = blockIdx.x, h = blockIdx.y, j0 = (ident ? (int)blockIdx.z - zv : (int)blockIdx.z) * GR_COLS;
   if (ident) m = n;
   const bool values = !ident;
@@ -111,11 +117,12 @@ gated_state_scan_kernel(const TI* __restrict__ x, int ld, int oq, int ok, int ov
     for (int u = 0; u < PERV; ++u) {
       const int idx = tid + u * 256;
       const int tt = idx / GR_COLS, c = idx - tt * GR_COLS;
-      rv[u] = (values && idx < nb * GR_COLS && j0 + c < m) ? to_f32(x[(size_t)(tb + tt) * ld + ov + h * m + j0 + c]) : 0.f;
+      rv[u] = (values && idx < nb * GR_COLS && j0 + c < mv) ? to_f32(x[(size_t)(tb + tt) * ld + ov + h * mv + j0 + c]) : 0.f;
+      if (ones && values && j0 + c == mv) rv[u] = 1.f;
     }
     if (tid < nb) {
       if (!VEC) r1 = decay[(size_t)(tb + tid) * lda + oa + h];
-      if (DELTA) rb = beta[(size_t)(tb + tid) * ldb + ob + h];
+      if (STRENGTH) rb = beta[(size_t)(tb + tid) * ldb + ob + h];
     }
   };
   auto put = [&](int tb) {
@@ -138,7 +145,7 @@ gated_state_scan_kernel(const TI* __restrict__ x, int ld, int oq, int ok, int ov
     }
     if (tid < nb) {
       if (!VEC) a1[tid] = r1;
-      if (DELTA) bs[tid] = rb;
+      if (STRENGTH) bs[tid] = rb;
     }
   };
   // the places of rows beyond n (where n is no multiple of 16) are written here once and never again: such a row of
@@ -163,7 +170,7 @@ gated_state_scan_kernel(const TI* __restrict__ x, int ld, int oq, int ok, int ov
     }
     t.v = vs[tt][jl];
     t.a1 = VEC ? 0.f : a1[tt];
-    t.b = DELTA ? bs[tt] : 0.f;
+    t.b = STRENGTH ? bs[tt] : 0.f;
   };
   auto advance = [&](const Tok& t, int row) __attribute__((always_inline)) {
     float u = t.v;
@@ -178,6 +185,7 @@ gated_state_scan_kernel(const TI* __restrict__ x, int ld, int oq, int ok, int ov
       }
     }
     if (DELTA) u = t.b * (u - gr_sum16((p0 + p1) + (p2 + p3)));
+    else if (STRENGTH) u *= t.b;
     p0 = p1 = p2 = p3 = 0.f;
 #pragma unroll
     for (int r = 0; r < RMAX; ++r) {
@@ -219,18 +227,21 @@ gated_state_scan_kernel(const TI* __restrict__ x, int ld, int oq, int ok, int ov
 extern "C" int gs_gated_state_scan(const void* x, int dtype, int ld, int oq, int ok, int ov, int qk_heads, float q_scale,
                                    const float* decay, int lda, int oa, int per_channel, const float* beta, int ldb,
                                    int ob, float* state, const int* q_start, const int* slots, float* out, int nseq,
-                                   int H, int n, int m, float* seg_m, float* seg_d, hipStream_t stream) {
+                                   int H, int n, int m, float* seg_m, float* seg_d, int delta, int ones, hipStream_t stream) {
   GS_REQUIRE(nseq >= 0 && H > 0 && n > 0 && m > 0, "gated_state_scan: bad sizes nseq=%d H=%d n=%d m=%d", nseq, H, n, m);
   GS_REQUIRE(n <= 256, "gated_state_scan: keys of %d features, the kernel holds up to 256", n);
   GS_REQUIRE(qk_heads > 0 && H % qk_heads == 0, "gated_state_scan: %d heads do not share %d queries and keys evenly", H,
              qk_heads);
   GS_REQUIRE(H <= 65535 && m <= 1000000, "gated_state_scan: too many heads or value columns");
   // (out null: the states alone are wanted)
-  GS_REQUIRE(!((seg_m || seg_d) && out) && !(seg_m && seg_d) && !(seg_d && beta),
+  delta = delta && beta;
+  GS_REQUIRE(ones == 0 || (ones == 1 && m >= 2 && !delta), "gated_state_scan: a column of ones goes with stored columns and no delta rule");
+  GS_REQUIRE(!((seg_m || seg_d) && out) && !(seg_m && seg_d) && !(seg_d && delta),
              "gated_state_scan: what a run does to a state is a matrix with the delta rule or a diagonal without, and comes without outputs");
-  GS_REQUIRE(oq >= 0 && ok >= 0 && ov >= 0 && oq + qk_heads * n <= ld && ok + qk_heads * n <= ld && ov + H * m <= ld,
+  GS_REQUIRE(oq >= 0 && ok >= 0 && ov >= 0 && oq + qk_heads * n <= ld && ok + qk_heads * n <= ld && ov + H * (m - ones) <= ld,
              "gated_state_scan: q, k or v lie outside the rows of %d", ld);
   GS_REQUIRE(decay && oa >= 0 && oa + (per_channel ? H * n : H) <= lda, "gated_state_scan: the decays lie outside their rows of %d", lda);
+  GS_REQUIRE(!(beta && per_channel) || delta, "gated_state_scan: write strengths without the delta rule go with a decay a head");
   GS_REQUIRE(!beta || (ob >= 0 && ob + H <= ldb), "gated_state_scan: the write strengths lie outside their rows of %d", ldb);
   if (nseq == 0) return 0;
   dim3 grid(nseq, H, (m + GR_COLS - 1) / GR_COLS + (seg_m ? (n + GR_COLS - 1) / GR_COLS : 0));
@@ -238,17 +249,18 @@ extern "C" int gs_gated_state_scan(const void* x, int dtype, int ld, int oq, int
   const int rep = H / qk_heads;
 #define GR_RUN(TI, R, V, D)                                                                                         \
   gated_state_scan_kernel<TI, R, V, D><<<grid, 256, 0, stream>>>((const TI*)x, ld, oq, ok, ov, rep, q_scale, decay, \
-                                                                 lda, oa, beta, ldb, ob, state, q_start, slots, out, H, n, m, seg_m, seg_d)
+                                                                 lda, oa, beta, ldb, ob, state, q_start, slots, out, H, n, m, seg_m, seg_d, ones)
 #define GR_RUN_R(TI, V, D)                   \
   if (n <= 32) GR_RUN(TI, 2, V, D);          \
   else if (n <= 64) GR_RUN(TI, 4, V, D);     \
   else if (n <= 128) GR_RUN(TI, 8, V, D);    \
   else GR_RUN(TI, 16, V, D)
 #define GR_RUN_T(TI)                                      \
-  if (per_channel && beta) { GR_RUN_R(TI, true, true); }  \
-  else if (per_channel) { GR_RUN_R(TI, true, false); }    \
-  else if (beta) { GR_RUN_R(TI, false, true); }           \
-  else { GR_RUN_R(TI, false, false); }
+  if (per_channel && delta) { GR_RUN_R(TI, true, 1); }    \
+  else if (per_channel) { GR_RUN_R(TI, true, 0); }        \
+  else if (delta) { GR_RUN_R(TI, false, 1); }             \
+  else if (beta) { GR_RUN_R(TI, false, 2); }              \
+  else { GR_RUN_R(TI, false, 0); }
   if (dtype == GS_F32) {
     GR_RUN_T(float)
   } else if (dtype == GS_BF16) {

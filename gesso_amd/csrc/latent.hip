@@ -63,7 +63,7 @@ extern "C" int gs_latent_prep(const void* down, int dtype, int ld, int q_off, in
                               int page_size, void* cache, void* a_out, int write_kv, int ntok, hipStream_t stream) {
   GS_REQUIRE(ntok >= 0 && q_rank > 0 && c > 0 && r >= 0 && r % 2 == 0, "latent_prep: bad sizes T=%d q_rank=%d c=%d r=%d",
              ntok, q_rank, c, r);
-  GS_REQUIRE(q_off >= 0 && kv_off >= 0 && q_off + q_rank <= ld && kv_off + c + r <= ld,
+  GS_REQUIRE(q_off >= 0 && kv_off >= 0 && q_off + q_rank <= ld && (!write_kv || (kvw && kv_off + c + r <= ld)),
              "latent_prep: columns %d+%d, %d+%d+%d outside rows of %d", q_off, q_rank, kv_off, c, r, ld);
   GS_REQUIRE(page_size > 0 && max_blocks > 0, "latent_prep: bad page_size/max_blocks");
   if (ntok == 0) return 0;
@@ -314,6 +314,8 @@ extern "C" int gs_heads_product(const void* X, int x_dtype, int ldx, int hx, con
 //
 //   s_u = (q~ . row_u) * scale over all D = c + r columns;  o = sum_u softmax(s)_u row_u[:c]
 //
+// With `sinks` (one float32 a head) the softmax's denominator has one more term, exp(sinks[h]), which has no row.
+//
 // qa (T, H D); out (T, H c); cache (pages, page_size, D).
 #define LAT_MAX_C 2048
 
@@ -321,7 +323,8 @@ template <typename T>
 __global__ void attention_latent_kernel(const T* __restrict__ qa, const T* __restrict__ cache,
                                         const int* __restrict__ positions, const int* __restrict__ seq_of_token,
                                         const int* __restrict__ block_table, int max_blocks, int page_size, int window,
-                                        float scale, T* __restrict__ out, int H, int c, int D) {
+                                        float scale, T* __restrict__ out, int H, int c, int D,
+                                        const float* __restrict__ sinks) {
   extern __shared__ float qs[];      // D floats
   __shared__ float ps[64];
   __shared__ long rowoff[64];
@@ -331,7 +334,7 @@ __global__ void attention_latent_kernel(const T* __restrict__ qa, const T* __res
   for (int j = lane; j < D; j += 64) qs[j] = to_f32(qa[((size_t)t * H + h) * D + j]);
   __syncthreads();
   const int lo = window > 0 ? (pos - window + 1 > 0 ? pos - window + 1 : 0) : 0;
-  float m = -INFINITY, l = 0.f;
+  float m = sinks ? sinks[h] : -INFINITY, l = sinks ? 1.f : 0.f;      // the sink's own term: its score is stored as it counts
   float acc[LAT_MAX_C / 64];
 #pragma unroll
   for (int i = 0; i < LAT_MAX_C / 64; ++i) acc[i] = 0.f;
@@ -376,7 +379,7 @@ __global__ void attention_latent_kernel(const T* __restrict__ qa, const T* __res
 
 extern "C" int gs_attention_latent(const void* qa, const void* cache, int dtype, const int* positions,
                                    const int* seq_of_token, const int* block_table, int max_blocks, int page_size,
-                                   int window, float scale, void* out, int ntok, int H, int c, int r,
+                                   int window, float scale, void* out, int ntok, int H, int c, int r, const float* sinks,
                                    hipStream_t stream) {
   GS_REQUIRE(ntok >= 0 && H > 0 && c > 0 && r >= 0, "attention_latent: bad sizes T=%d H=%d c=%d r=%d", ntok, H, c, r);
   GS_REQUIRE(c <= LAT_MAX_C && c + r <= 12288, "attention_latent: latent rows of %d + %d above the kernel's limit", c, r);
@@ -388,11 +391,11 @@ extern "C" int gs_attention_latent(const void* qa, const void* cache, int dtype,
   if (dtype == GS_F32)
     attention_latent_kernel<float><<<grid, 64, D * sizeof(float), stream>>>(
         (const float*)qa, (const float*)cache, positions, seq_of_token, block_table, max_blocks, page_size, window, scale,
-        (float*)out, H, c, D);
+        (float*)out, H, c, D, sinks);
   else if (dtype == GS_BF16)
     attention_latent_kernel<bf16><<<grid, 64, D * sizeof(float), stream>>>(
         (const bf16*)qa, (const bf16*)cache, positions, seq_of_token, block_table, max_blocks, page_size, window, scale,
-        (bf16*)out, H, c, D);
+        (bf16*)out, H, c, D, sinks);
   else
     GS_REQUIRE(false, "attention_latent: unknown dtype %d", dtype);
   GS_LAUNCH_CHECK("attention_latent");

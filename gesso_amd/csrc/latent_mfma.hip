@@ -17,7 +17,8 @@
 //
 // The query at position p sees rows lo..p of its sequence, lo = 0 or p - window + 1; a block walks from the oldest row
 // any of its queries sees to its last query's own, each row masked per query.  Rows past the block's last are staged
-// as zeros (their pages may belong to nobody).
+// as zeros (their pages may belong to nobody).  With `sinks` (one float32 a head) the softmax's denominator has one more
+// term, exp(sinks[h]), which has no row: the running maximum and sum start from it.
 #include "common.h"
 
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8_t;
@@ -35,7 +36,7 @@ __global__ __launch_bounds__(256) void attention_latent_mfma_kernel(
     const int* __restrict__ tile_seq, const int* __restrict__ tile_row, const int* __restrict__ tile_n,
     const int* __restrict__ block_table, int max_blocks, int page_size, int window, float scale,
     bf16* __restrict__ out, float* __restrict__ part_o, float* __restrict__ part_ml, int nsplit, int rows_total, int H,
-    int HB, int c, int D) {
+    int HB, int c, int D, const float* __restrict__ sinks) {
   constexpr int DK = CT / 2 + 2;
   constexpr int NB = KSTEP / 16, NC = KSTEP / 32, VROW = KSTEP + 4;
   extern __shared__ __attribute__((aligned(16))) unsigned char lds[];
@@ -80,6 +81,10 @@ __global__ __launch_bounds__(256) void attention_latent_mfma_kernel(
 #pragma unroll
   for (int dt = 0; dt < CT; ++dt) acc[dt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
   float mrun = -INFINITY, lrun = 0.f;
+  if (sinks && blockIdx.z == 0) {                    // the sink's own term, counted by the first of the blocks that share a row's keys
+    mrun = sinks[head] * LM_LOG2E;
+    lrun = 1.f;
+  }
   const float sc = scale * LM_LOG2E;
   const int kmax = pos0 + nt - 1;
   const int kmin = window > 0 ? (pos0 - window + 1 > 0 ? pos0 - window + 1 : 0) : 0;
@@ -293,7 +298,7 @@ extern "C" int gs_attention_latent_mfma_tokens(int H) {
 extern "C" int gs_attention_latent_mfma(const void* qa, const void* cache, const int* positions, const int* tile_seq,
                                         const int* tile_row, const int* tile_n, int ntiles, const int* block_table,
                                         int max_blocks, int page_size, int window, float scale, void* out, int H, int c,
-                                        int r, int nsplit, float* part_o, float* part_ml, int ntok, hipStream_t stream) {
+                                        int r, int nsplit, float* part_o, float* part_ml, int ntok, const float* sinks, hipStream_t stream) {
   GS_REQUIRE(gs_attention_latent_mfma_supports(H, c, r), "attention_latent_mfma: sizes H=%d c=%d r=%d are not taken", H, c, r);
   GS_REQUIRE(ntiles >= 0 && page_size > 0 && max_blocks > 0 && window >= 0, "attention_latent_mfma: bad tiles/page_size/max_blocks/window");
   GS_REQUIRE((tile_seq == nullptr) == (tile_row == nullptr) && (tile_seq == nullptr) == (tile_n == nullptr),
@@ -310,7 +315,7 @@ extern "C" int gs_attention_latent_mfma(const void* qa, const void* cache, const
     const size_t lds = (size_t)64 * (Dp + 8) * 2 + (size_t)((c + 63) & ~63) * (64 + 4) * 2;
     attention_latent_mfma_kernel<8, 64><<<grid, 256, lds, stream>>>(
         (const bf16*)qa, (const bf16*)cache, positions, tile_seq, tile_row, tile_n, block_table, max_blocks, page_size,
-        window, scale, (bf16*)out, part_o, part_ml, nsplit, rows_total, H, HB, c, D);
+        window, scale, (bf16*)out, part_o, part_ml, nsplit, rows_total, H, HB, c, D, sinks);
   } else if (c <= 256 && D <= 32 * (16 / 2 + 2)) {
     // latents up to 256: half the accumulators of the widest form, so steps of 64 rows fit
     const size_t lds = (size_t)64 * (Dp + 8) * 2 + (size_t)((c + 63) & ~63) * (64 + 4) * 2;
@@ -324,7 +329,7 @@ extern "C" int gs_attention_latent_mfma(const void* qa, const void* cache, const
     GS_REQUIRE(lds <= 96 * 1024, "attention_latent_mfma: %zu bytes of LDS", lds);
     attention_latent_mfma_kernel<16, 64><<<grid, 256, lds, stream>>>(
         (const bf16*)qa, (const bf16*)cache, positions, tile_seq, tile_row, tile_n, block_table, max_blocks, page_size,
-        window, scale, (bf16*)out, part_o, part_ml, nsplit, rows_total, H, HB, c, D);
+        window, scale, (bf16*)out, part_o, part_ml, nsplit, rows_total, H, HB, c, D, sinks);
   } else {
     const size_t lds = (size_t)32 * (Dp + 8) * 2 + (size_t)((c + 63) & ~63) * (32 + 4) * 2;
     static bool raised = false;
@@ -337,7 +342,7 @@ extern "C" int gs_attention_latent_mfma(const void* qa, const void* cache, const
     GS_REQUIRE(lds <= 96 * 1024, "attention_latent_mfma: %zu bytes of LDS", lds);
     attention_latent_mfma_kernel<32, 32><<<grid, 256, lds, stream>>>(
         (const bf16*)qa, (const bf16*)cache, positions, tile_seq, tile_row, tile_n, block_table, max_blocks, page_size,
-        window, scale, (bf16*)out, part_o, part_ml, nsplit, rows_total, H, HB, c, D);
+        window, scale, (bf16*)out, part_o, part_ml, nsplit, rows_total, H, HB, c, D, sinks);
   }
   GS_LAUNCH_CHECK("attention_latent_mfma");
   if (nsplit > 1) {

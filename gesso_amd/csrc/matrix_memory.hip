@@ -1,0 +1,124 @@
+// What a matrix memory with exponential gates computes around its recurrence (gated_recurrence.hip walks the memory itself).
+//
+// exp_gates: per token and head, from the products z (T, ldz) float32 (the input gate's at [oi + h], the forget gate's at
+// [of + h]), biases added,
+//   i = cap tanh(zi / cap),   f = log sigmoid(cap tanh(zf / cap))
+//   p_t = max(f_t + p_(t-1), i_t)                        a running maximum, the request's own, kept in its slot
+//   gates[t, h] = exp(f + p_(t-1) - p_t)                 what the memory keeps
+//   gates[t, H + h] = exp(i - p_t)                       with what the token is written
+//   gates[t, 2 H + h] = exp(-p_t)                        the least the output is divided by
+// A wavefront per (sequence, head), 64 tokens a turn: a token takes the maximum from p to max(p + f, i), and such maps
+// compose, (f1, i1) then (f2, i2) = (f1 + f2, max(i1 + f2, i2)), so six steps between lanes give every token's p.
+//
+// memory_outnorm: o (T, H (m + 1)) float32, a head's m columns and then the column whose values are ones (n . q):
+//   u = o / (max(|n . q|, exp(-p)) + 1e-6);   out = u / sqrt(mean(u^2) + eps) * w * sigmoid(gate)      per head
+#include "common.h"
+
+__global__ void __launch_bounds__(256)
+exp_gates_kernel(const float* __restrict__ z, int ldz, int oi, int of, const float* __restrict__ bi,
+                 const float* __restrict__ bf, float cap, float* __restrict__ peak, const int* __restrict__ q_start,
+                 const int* __restrict__ slots, float* __restrict__ gates, int H) {
+  const int lane = threadIdx.x & 63, h = blockIdx.y * 4 + (threadIdx.x >> 6), seq = blockIdx.x;
+  if (h >= H) return;
+  const int t0 = q_start[seq], t1 = q_start[seq + 1];
+  if (t1 <= t0) return;
+  float* own = peak + (size_t)slots[seq] * H + h;
+  float p = *own;
+  const float b_i = bi[h], b_f = bf[h];
+  for (int tb = t0; tb < t1; tb += 64) {
+    const int t = tb + lane;
+    const bool live = t < t1;
+    float f = 0.f, i = -INFINITY;                    // (a lane without a token: the map that changes nothing)
+    if (live) {
+      const float zi = z[(size_t)t * ldz + oi + h] + b_i, zf = z[(size_t)t * ldz + of + h] + b_f;
+      i = cap * tanhf(zi / cap);
+      const float u = cap * tanhf(zf / cap);
+      f = fminf(u, 0.f) - log1pf(expf(-fabsf(u)));
+    }
+    float F = f, M = i;
+#pragma unroll
+    for (int o = 1; o < 64; o <<= 1) {
+      const float Fb = __shfl_up(F, o, 64), Mb = __shfl_up(M, o, 64);
+      if (lane >= o) {
+        M = fmaxf(Mb + F, M);
+        F += Fb;
+      }
+    }
+    const float now = fmaxf(p + F, M);
+    const float up = __shfl_up(now, 1, 64), before = lane == 0 ? p : up;
+    if (live) {
+      float* g = gates + (size_t)t * 3 * H + h;
+      g[0] = expf(f + before - now);
+      g[H] = expf(i - now);
+      g[2 * H] = expf(-now);
+    }
+    p = __shfl(now, t1 - tb < 64 ? t1 - tb - 1 : 63, 64);
+  }
+  if (lane == 0) *own = p;
+}
+
+extern "C" int gs_exp_gates(const float* z, int ldz, int oi, int of, const float* bi, const float* bf, float cap, float* peak,
+                            const int* q_start, const int* slots, float* gates, int nseq, int H, hipStream_t stream) {
+  GS_REQUIRE(nseq >= 0 && H > 0 && H <= 4 * 65535, "exp_gates: bad sizes nseq=%d H=%d", nseq, H);
+  GS_REQUIRE(oi >= 0 && of >= 0 && oi + H <= ldz && of + H <= ldz, "exp_gates: the gates' products lie outside the rows of %d", ldz);
+  GS_REQUIRE(cap > 0.f, "exp_gates: the cap must be positive");
+  if (nseq == 0) return 0;
+  exp_gates_kernel<<<dim3(nseq, gs_ceil_div(H, 4)), 256, 0, stream>>>(z, ldz, oi, of, bi, bf, cap, peak, q_start, slots, gates, H);
+  GS_LAUNCH_CHECK("exp_gates");
+  return 0;
+}
+
+// One block per token, a wavefront per head in turn; a lane's columns are c = lane, lane + 64, ...: up to MM_KEEP of them
+// stay in registers between the two passes.
+#define MM_KEEP 8
+template <typename TG, typename TO>
+__global__ void __launch_bounds__(256)
+memory_outnorm_kernel(const float* __restrict__ o, const float* __restrict__ gates, const TG* __restrict__ rows, int ldr,
+                      int og, const float* __restrict__ w, float eps, TO* __restrict__ out, int H, int m) {
+  const int t = blockIdx.x, lane = threadIdx.x & 63, nw = blockDim.x >> 6;
+  for (int h = threadIdx.x >> 6; h < H; h += nw) {
+    const float* row = o + ((size_t)t * H + h) * (m + 1);
+    const TG* gt = rows + (size_t)t * ldr + og + (size_t)h * m;
+    const float inv_den = 1.0f / (fmaxf(fabsf(row[m]), gates[(size_t)t * 3 * H + 2 * H + h]) + 1e-6f);
+    float keep[MM_KEEP], ss = 0.f;
+#pragma unroll
+    for (int u = 0; u < MM_KEEP; ++u) {
+      const int c = lane + 64 * u;
+      keep[u] = c < m ? row[c] * inv_den : 0.f;
+      ss += keep[u] * keep[u];
+    }
+    for (int c = lane + 64 * MM_KEEP; c < m; c += 64) {
+      const float v = row[c] * inv_den;
+      ss += v * v;
+    }
+    const float inv = norm_inverse(wave_sum(ss), (float)m, eps);
+    TO* dst = out + ((size_t)t * H + h) * m;
+    const float* wh = w + (size_t)h * m;
+#pragma unroll
+    for (int u = 0; u < MM_KEEP; ++u) {
+      const int c = lane + 64 * u;
+      if (c < m) dst[c] = from_f32<TO>(keep[u] * inv * wh[c] / (1.0f + expf(-to_f32(gt[c]))));
+    }
+    for (int c = lane + 64 * MM_KEEP; c < m; c += 64)
+      dst[c] = from_f32<TO>(row[c] * inv_den * inv * wh[c] / (1.0f + expf(-to_f32(gt[c]))));
+  }
+}
+
+extern "C" int gs_memory_outnorm(const float* o, const float* gates, const void* rows, int rows_dtype, int ldr, int og,
+                                 const float* w, float eps, void* out, int out_dtype, int T, int H, int m,
+                                 hipStream_t stream) {
+  GS_REQUIRE(T >= 0 && H > 0 && m > 0 && og >= 0 && og + H * m <= ldr, "memory_outnorm: bad sizes T=%d H=%d m=%d, or a gate outside the rows of %d", T, H, m, ldr);
+  GS_REQUIRE(eps > 0.f, "memory_outnorm: eps must be positive");
+  if (T == 0) return 0;
+  const int threads = H >= 4 ? 256 : 64 * H;
+  if (rows_dtype == GS_F32 && out_dtype == GS_F32)
+    memory_outnorm_kernel<float, float><<<T, threads, 0, stream>>>(o, gates, (const float*)rows, ldr, og, w, eps, (float*)out, H, m);
+  else if (rows_dtype == GS_BF16 && out_dtype == GS_BF16)
+    memory_outnorm_kernel<bf16, bf16><<<T, threads, 0, stream>>>(o, gates, (const bf16*)rows, ldr, og, w, eps, (bf16*)out, H, m);
+  else if (rows_dtype == GS_F32 && out_dtype == GS_BF16)
+    memory_outnorm_kernel<float, bf16><<<T, threads, 0, stream>>>(o, gates, (const float*)rows, ldr, og, w, eps, (bf16*)out, H, m);
+  else
+    GS_REQUIRE(false, "memory_outnorm: unknown dtypes %d %d", rows_dtype, out_dtype);
+  GS_LAUNCH_CHECK("memory_outnorm");
+  return 0;
+}

@@ -493,7 +493,7 @@ def attention_decode_maps(rows, kcache, vcache, positions, block_table, page_siz
 
 _ACTS = {None: 0, "none": 0, "silu": 1}
 _GATES = {"sigmoid": 0, "silu": 1}
-GATED_ACTS = {"silu": 0, "gelu_tanh": 1, "gelu": 2}
+GATED_ACTS = {"silu": 0, "gelu_tanh": 1, "gelu": 2, "relu_squared": 3}
 LINEAR_ATTENTION_MAX_KEY = 512
 LINEAR_ATTENTION_CHUNKS_MAX_KEY = 128
 
@@ -1224,13 +1224,15 @@ def latent_prep(down, q_off, q_rank, kv_off, c, r, q_weight, kv_weight, eps, cos
     """Per token of ``down (T, ld)``: the columns ``[q_off, q_off + q_rank)`` RMS-normed with ``q_weight`` are
     returned as ``(T, q_rank)``; the columns ``[kv_off, kv_off + c)`` RMS-normed with ``kv_weight`` and the ``r``
     columns behind them, rotated by the token's position, are written into the token's cache row ``[c | r]``.
-    ``cache (pages, 1, page_size, c + r)``."""
+    ``cache (pages, 1, page_size, c + r)``.  ``write_kv = False``: the query part alone (the cache is another's, the
+    rows hold no such columns)."""
     _dev(down, q_weight, kv_weight, positions, seq_of_token, block_table, cache)
     T, ld = down.shape
     _need(cache.dtype == down.dtype and cache.dim() == 4 and cache.shape[1:] == (1, page_size, c + r),
           "latent_prep: the cache is (pages, 1, page_size, c + r) in the activations' type")
-    _need(q_weight.dtype == torch.float32 and q_weight.shape == (q_rank,) and kv_weight.dtype == torch.float32
-          and kv_weight.shape == (c,), "latent_prep: norm weights are float32 (q_rank,), (c,)")
+    _need(q_weight.dtype == torch.float32 and q_weight.shape == (q_rank,)
+          and (not write_kv or (kv_weight.dtype == torch.float32 and kv_weight.shape == (c,))),
+          "latent_prep: norm weights are float32 (q_rank,), (c,)")
     if r:
         _dev(cos, sin)
         _need(cos.dtype == torch.float32 and sin.shape == cos.shape and cos.dim() == 2 and cos.shape[1] == r // 2,
@@ -1285,10 +1287,12 @@ def heads_product(x, hx: int, w, y, hy: int, K: int, gate=None, gate_each: bool 
 
 
 def attention_latent(qa, cache, positions, seq_of_token, block_table, page_size, window, scale, H, c, r, ntok,
-                     out: torch.Tensor = None) -> torch.Tensor:
+                     out: torch.Tensor = None, sinks=None) -> torch.Tensor:
     """Attention of ``qa (T, H (c + r))`` over cached rows ``[c | r]``: scores over all ``c + r`` columns, the output
-    ``(T, H c)`` a softmax-weighted sum of the rows' first ``c`` columns.  Any sizes, float32 arithmetic."""
-    _dev(qa, cache, positions, seq_of_token, block_table, out)
+    ``(T, H c)`` a softmax-weighted sum of the rows' first ``c`` columns.  ``sinks (H,)`` float32: the softmax's
+    denominator has one more term ``exp(sinks[h])``.  Any sizes, float32 arithmetic."""
+    _dev(qa, cache, positions, seq_of_token, block_table, out, sinks)
+    _need(sinks is None or (sinks.dtype == torch.float32 and sinks.shape == (H,)), "attention_latent: sinks must be float32 (H,)")
     _need(qa.shape == (ntok, H * (c + r)) and cache.dtype == qa.dtype, "attention_latent: qa is (T, H (c + r)) in the cache's type")
     _need(cache.dim() == 4 and cache.shape[1:] == (1, page_size, c + r), "attention_latent: the cache is (pages, 1, page_size, c + r)")
     _i32(positions, ntok, "positions")
@@ -1299,7 +1303,7 @@ def attention_latent(qa, cache, positions, seq_of_token, block_table, page_size,
     _need(out.shape == (ntok, H * c) and out.dtype == qa.dtype, "attention_latent: out has the wrong shape or type")
     _check(lib().gs_attention_latent(_p(qa), _p(cache), _dt(qa), _p(positions), _p(seq_of_token), _p(block_table),
                                      block_table.shape[1], page_size, window or 0, float(scale), _p(out), ntok, H, c, r,
-                                     _stream()))
+                                     _p(sinks), _stream()))
     return out
 
 
@@ -1366,12 +1370,13 @@ def _latent_workspace(device, rows: int, c: int, nsplit: int):
 
 
 def attention_latent_mfma(qa, cache, positions, tiles, block_table, page_size, window, scale, H, c, r, ntok,
-                          out: torch.Tensor = None, nsplit: int = 1) -> torch.Tensor:
+                          out: torch.Tensor = None, nsplit: int = 1, sinks=None) -> torch.Tensor:
     """:func:`attention_latent` on the matrix cores (bfloat16).  ``tiles``: int32 ``(3, n)``, the sequence, first row
     and token count (at most :func:`attention_latent_mfma_tokens`) of every tile of consecutive tokens of one
     sequence; None: sequence ``i`` brings the single token ``i``.  ``nsplit`` > 1: as many blocks share a tile's keys out
     between them in runs of whole steps, and a second kernel adds their shares."""
-    _dev(qa, cache, positions, block_table, out, tiles)
+    _dev(qa, cache, positions, block_table, out, tiles, sinks)
+    _need(sinks is None or (sinks.dtype == torch.float32 and sinks.shape == (H,)), "attention_latent_mfma: sinks must be float32 (H,)")
     _need(1 <= nsplit <= 64, "attention_latent_mfma: 1 to 64 parts")
     _need(qa.dtype == torch.bfloat16 and cache.dtype == torch.bfloat16, "attention_latent_mfma takes bfloat16")
     _need(qa.shape == (ntok, H * (c + r)), "attention_latent_mfma: qa is (T, H (c + r))")
@@ -1392,7 +1397,7 @@ def attention_latent_mfma(qa, cache, positions, tiles, block_table, page_size, w
     part_o, part_ml = _latent_workspace(qa.device, ntok * H, c, nsplit) if nsplit > 1 else (None, None)
     _check(lib().gs_attention_latent_mfma(_p(qa), _p(cache), _p(positions), _p(rows[0]), _p(rows[1]), _p(rows[2]), n,
                                           _p(block_table), block_table.shape[1], page_size, window or 0, float(scale),
-                                          _p(out), H, c, r, nsplit, _p(part_o), _p(part_ml), ntok, _stream()))
+                                          _p(out), H, c, r, nsplit, _p(part_o), _p(part_ml), ntok, _p(sinks), _stream()))
     return out
 
 
@@ -1706,16 +1711,17 @@ GATED_STATE_MAX_KEY = 256
 
 def gated_state_scan(x, oq: int, ok: int, ov: int, H: int, qk_heads: int, n: int, m: int, decay, oa: int,
                      per_channel: bool, state, q_start, slots, nseq: int, q_scale: float = 1.0, beta=None, ob: int = 0,
-                     out: torch.Tensor = None, seg_m=None, seg_d=None) -> torch.Tensor:
-    """Per sequence and head ``S <- diag(a_t) S; u = beta_t (v_t - S^T k_t)`` (``u = v_t`` without ``beta``);
-    ``S <- S + k_t u^T; o_t = S^T (q_scale q_t)``.
+                     out: torch.Tensor = None, seg_m=None, seg_d=None, delta: bool = True, ones: bool = False) -> torch.Tensor:
+    """Per sequence and head ``S <- diag(a_t) S; u = beta_t (v_t - S^T k_t)`` (``u = v_t`` without ``beta``, ``beta_t v_t``
+    with ``beta`` and ``delta = False``); ``S <- S + k_t u^T; o_t = S^T (q_scale q_t)``.  ``ones``: a head's last value
+    column is not stored, its values are all one (v then has ``m - 1`` columns a head).
 
     ``x (T, ld)`` float32 or bfloat16 holds q of head ``h`` at ``[oq + (h // (H / qk_heads)) n, ...)``, k likewise from
     ``ok``, v at ``[ov + h m, ...)``.  ``decay`` float32 rows: ``a_t`` of head ``h`` at
     ``[oa + h]``, or with ``per_channel`` one a key channel at ``[oa + h n, ...)``.  ``beta`` float32 rows with head ``h``
     at ``[ob + h]``.  ``state (slots, H, n, m)`` float32 is read and advanced.  Returns ``(T, H m)`` float32.
 
-    ``seg_m (slots, H, n, n)`` or, without ``beta``, ``seg_d (slots, H, n)`` float32: what the tokens do to a state, ``S -> M S
+    ``seg_m (slots, H, n, n)`` or, without the delta rule, ``seg_d (slots, H, n)`` float32: what the tokens do to a state, ``S -> M S
     + B``, instead of outputs: ``state`` is not read and receives ``B``, ``seg_m`` the matrices ``M`` (``seg_d`` their
     diagonals, the products of the decays); returns None."""
     _dev(x, decay, beta, state, q_start, slots, out, seg_m, seg_d)
@@ -1731,7 +1737,9 @@ def gated_state_scan(x, oq: int, ok: int, ov: int, H: int, qk_heads: int, n: int
     _i32(slots, nseq, "slots")
     _need(seg_m is None or (seg_d is None and seg_m.dtype == torch.float32 and seg_m.shape == state.shape[:3] + (n,)),
           "gated_state_scan: the runs' matrices are float32 (slots, H, n, n)")
-    _need(seg_d is None or (beta is None and seg_d.dtype == torch.float32 and seg_d.shape == state.shape[:3]),
+    delta = delta and beta is not None
+    _need(not (delta and ones), "gated_state_scan: a column of ones goes without the delta rule")
+    _need(seg_d is None or (not delta and seg_d.dtype == torch.float32 and seg_d.shape == state.shape[:3]),
           "gated_state_scan: the runs' diagonals are float32 (slots, H, n), without the delta rule")
     if seg_m is None and seg_d is None:
         if out is None:
@@ -1741,7 +1749,8 @@ def gated_state_scan(x, oq: int, ok: int, ov: int, H: int, qk_heads: int, n: int
         out = None
     _check(lib().gs_gated_state_scan(_p(x), _dt(x), ld, oq, ok, ov, qk_heads, float(q_scale), _p(decay), decay.shape[1], oa,
                                      1 if per_channel else 0, _p(beta), beta.shape[1] if beta is not None else 0, ob,
-                                     _p(state), _p(q_start), _p(slots), _p(out), nseq, H, n, m, _p(seg_m), _p(seg_d), _stream()))
+                                     _p(state), _p(q_start), _p(slots), _p(out), nseq, H, n, m, _p(seg_m), _p(seg_d),
+                                     1 if delta else 0, 1 if ones else 0, _stream()))
     return out
 
 
@@ -1762,7 +1771,7 @@ def state_segment_tables(q_lens, seg_len: int, device):
 
 def gated_state_scan_segments(x, oq: int, ok: int, ov: int, H: int, qk_heads: int, n: int, m: int, decay, oa: int,
                               per_channel: bool, state, q_lens, slots, seg_len: int, q_scale: float = 1.0, beta=None,
-                              ob: int = 0) -> torch.Tensor:
+                              ob: int = 0, delta: bool = True, ones: bool = False) -> torch.Tensor:
     """:func:`gated_state_scan` with the portions (``q_lens``: tokens of each sequence, on the host) cut into segments of
     ``seg_len`` tokens that run side by side.  Over a segment the state goes ``S -> M S + B``: one launch of the kernel gives
     every segment's ``B`` (from a state of zeros) and ``M`` (from the identity, every value zero; without the delta rule the
@@ -1775,11 +1784,12 @@ def gated_state_scan_segments(x, oq: int, ok: int, ov: int, H: int, qk_heads: in
     _i32(slots, nseq, "slots")
     _need(state.dtype == torch.float32 and state.dim() == 4 and state.shape[1:] == (H, n, m), "gated_state_scan: state must be float32 (slots, H, n, m)")
     B, first = torch.empty((2, nseg, H, n, m), dtype=torch.float32, device=x.device)
-    M = torch.empty((nseg, H, n, n) if beta is not None else (nseg, H, n), dtype=torch.float32, device=x.device)
+    delta = delta and beta is not None
+    M = torch.empty((nseg, H, n, n) if delta else (nseg, H, n), dtype=torch.float32, device=x.device)
     args = (x, oq, ok, ov, H, qk_heads, n, m, decay, oa, per_channel)
-    kw = dict(q_scale=q_scale, beta=beta, ob=ob)
-    gated_state_scan(*args, B, seg_start, ids, nseg, **kw, **({"seg_m": M} if beta is not None else {"seg_d": M}))
-    chain = lib().gs_gated_state_chain if beta is not None else lib().gs_gated_state_chain_diagonal
+    kw = dict(q_scale=q_scale, beta=beta, ob=ob, delta=delta, ones=ones)
+    gated_state_scan(*args, B, seg_start, ids, nseg, **kw, **({"seg_m": M} if delta else {"seg_d": M}))
+    chain = lib().gs_gated_state_chain if delta else lib().gs_gated_state_chain_diagonal
     _check(chain(_p(M), _p(B), _p(first), _p(state), _p(seq_seg), _p(slots), nseq, H, n, m, _stream()))
     return gated_state_scan(*args, first, seg_start, ids, nseg, **kw)
 
@@ -1815,3 +1825,120 @@ def channel_decay(z, tau: float) -> torch.Tensor:
     _need(z.dtype == torch.float32, "channel_decay: float32 values")
     _check(lib().gs_channel_decay(_p(z), z.numel(), float(tau), _stream()))
     return z
+
+
+# ---------------------------------------------------------------------- a matrix memory with exponential gates
+
+def exp_gates(z, oi: int, of: int, bias_i, bias_f, cap: float, peak, q_start, slots, nseq: int, H: int) -> torch.Tensor:
+    """From float32 products ``z (T, ldz)`` (head ``h``'s input gate at ``[oi + h]``, its forget gate at ``[of + h]``):
+    ``i = cap tanh((z + b) / cap)``, ``f = log sigmoid(cap tanh((z + b) / cap))``, the running maximum
+    ``p_t = max(f + p_(t-1), i)`` from ``peak (slots, H)`` on, which it leaves there.  Returns float32 ``(T, 3 H)``:
+    ``exp(f + p_(t-1) - p_t)``, ``exp(i - p_t)``, ``exp(-p_t)``."""
+    _dev(z, bias_i, bias_f, peak, q_start, slots)
+    _need(z.dim() == 2 and z.dtype == torch.float32, "exp_gates: the products are float32 rows (T, ldz)")
+    for b in (bias_i, bias_f):
+        _need(b.dtype == torch.float32 and b.shape == (H,), "exp_gates: biases must be float32 (H,)")
+    _need(peak.dtype == torch.float32 and peak.dim() == 2 and peak.shape[1] == H, "exp_gates: the running maxima are float32 (slots, H)")
+    _i32(q_start, nseq + 1, "q_start")
+    _i32(slots, nseq, "slots")
+    gates = torch.empty((z.shape[0], 3 * H), dtype=torch.float32, device=z.device)
+    _check(lib().gs_exp_gates(_p(z), z.shape[1], oi, of, _p(bias_i), _p(bias_f), float(cap), _p(peak), _p(q_start), _p(slots),
+                              _p(gates), nseq, H, _stream()))
+    return gates
+
+
+def memory_outnorm(o, gates, rows, og: int, weight, eps: float, H: int, m: int, out_dtype) -> torch.Tensor:
+    """``o (T, H (m + 1))`` float32, each head's ``m`` columns and ``n . q`` behind them, ``gates`` as :func:`exp_gates`
+    leaves them: ``u = o / (max(|n . q|, exp(-p)) + 1e-6)``, ``u / sqrt(mean(u^2) + eps) * weight * sigmoid(gate)`` per
+    head; the gate stands in ``rows`` from column ``og`` on.  Returns ``(T, H m)`` in ``out_dtype``."""
+    _dev(o, gates, rows, weight)
+    T = o.shape[0]
+    _need(o.dtype == torch.float32 and o.shape == (T, H * (m + 1)), "memory_outnorm: o must be float32 (T, H (m + 1))")
+    _need(gates.dtype == torch.float32 and gates.shape == (T, 3 * H), "memory_outnorm: gates must be float32 (T, 3 H)")
+    _need(rows.dim() == 2 and rows.shape[0] == T, "memory_outnorm: the gate's rows are (T, ld)")
+    _need(weight.dtype == torch.float32 and weight.shape == (H * m,), "memory_outnorm: weight must be float32 (H m,)")
+    out = torch.empty((T, H * m), dtype=out_dtype, device=o.device)
+    _check(lib().gs_memory_outnorm(_p(o), _p(gates), _p(rows), _dt(rows), rows.shape[1], og, _p(weight), float(eps), _p(out),
+                                   _dt(out), T, H, m, _stream()))
+    return out
+
+
+NARROW_MAX_OUT = 64
+
+
+def narrow_ok(x, w: torch.Tensor) -> bool:
+    """Whether :func:`gemm_narrow` takes this product: bfloat16 rows against at most 64 weight rows, whole 16-byte pieces."""
+    return (isinstance(x, torch.Tensor) and x.dtype == torch.bfloat16 and w.dtype == torch.bfloat16 and x.dim() == 2
+            and w.shape[0] <= NARROW_MAX_OUT and w.shape[1] % 8 == 0 and x.stride(1) == 1 and x.data_ptr() % 16 == 0
+            and (x.shape[0] <= 1 or x.stride(0) % 8 == 0) and w.is_contiguous() and w.data_ptr() % 16 == 0)
+
+
+def gemm_narrow(x, w: torch.Tensor, out_dtype=torch.float32) -> torch.Tensor:
+    """``x @ w.T`` for many rows and at most 64 outputs (bfloat16 operands, float32 sums)."""
+    _need(narrow_ok(x, w) and x.is_cuda and x.shape[1] == w.shape[1], "gemm_narrow: bfloat16 rows against at most 64 weight rows")
+    M, K = x.shape
+    N = w.shape[0]
+    y = torch.empty((M, N), dtype=out_dtype, device=x.device)
+    _check(lib().gs_gemm_narrow(_p(x), x.stride(0) if M > 1 else K, _p(w), _p(y), _dt(y), N, M, N, K, _stream()))
+    return y
+
+
+# ---------------------------------------------------------------------- norms on both sides of a sub-layer, a token's own input
+
+class SeamNorm:
+    """A norm as :func:`norm_seam` takes it: ``("rms", w, eps)`` or ``("dyn_tanh", w, b, alpha)``."""
+
+    __slots__ = ("kind", "weight", "bias", "alpha", "eps")
+    KINDS = {"rms": 1, "dyn_tanh": 2}
+
+    def __init__(self, kind: str, weight, bias=None, alpha=None, eps: float = 0.0):
+        self.kind, self.weight, self.bias, self.alpha, self.eps = self.KINDS[kind], weight, bias, alpha, float(eps)
+
+    def check(self, H: int) -> None:
+        ts = [self.weight] if self.kind == 1 else [self.weight, self.bias]
+        _dev(*ts, self.alpha)
+        _need(all(t is not None and t.dtype == torch.float32 and t.shape == (H,) for t in ts), "norm_seam: a norm's vectors are float32 (H,)")
+        _need(self.kind == 1 or (self.alpha is not None and self.alpha.dtype == torch.float32 and self.alpha.numel() == 1),
+              "norm_seam: alpha is one float32 number on the device")
+
+    def args(self):
+        return self.kind, _p(self.weight), _p(self.bias), _p(self.alpha), self.eps
+
+
+_NO_SEAM_NORM = (0, None, None, None, 0.0)
+
+
+def norm_seam(res, y, post, mult: float, pre, rows_dtype=None, rows=None, out=None):
+    """``res += mult * post(y)`` (``y = None``: nothing), then ``pre(res)`` as rows of ``rows_dtype`` (None: no rows).
+    ``post``, ``pre``: a :class:`SeamNorm`, or None for the row as it is.  ``rows`` (int32) picks source rows; then
+    nothing is added."""
+    _dev(res, y, rows, out)
+    _need(res.dtype == torch.float32 and res.dim() == 2, "norm_seam: the residual stream is float32 (T, H)")
+    T, H = res.shape
+    _need(y is None or y.shape == res.shape, "norm_seam: y has the stream's shape")
+    for n in (post, pre):
+        if n is not None:
+            n.check(H)
+    n_out = T
+    if rows is not None:
+        _i32(rows, what="rows")
+        n_out = rows.numel()
+    if out is None and rows_dtype is not None:
+        out = torch.empty((n_out, H), dtype=rows_dtype, device=res.device)
+    _need(out is None or (out.shape == (n_out, H) and (rows_dtype is None or out.dtype == rows_dtype)), "norm_seam: out has the wrong shape or type")
+    _check(lib().gs_norm_seam(_p(res), _p(y), _dt(y) if y is not None else _dt(out), *(post.args() if post is not None else _NO_SEAM_NORM),
+                              float(mult), *(pre.args() if pre is not None else _NO_SEAM_NORM), _p(out),
+                              _dt(out) if out is not None else _dt(y), _p(rows), n_out, H, _stream()))
+    return out
+
+
+def side_gate(z, table, ids, offset: int, dim: int, width: int, out_dtype) -> torch.Tensor:
+    """``gelu_tanh(z[:, :dim]) * table[ids, offset : offset + dim]`` as rows ``(T, width)``, zeros in the spare columns."""
+    _dev(z, table, ids)
+    T = z.shape[0]
+    _need(z.dim() == 2 and z.shape[1] >= dim and table.dim() == 2, "side_gate: rows (T, >= dim) and a table (vocab, columns)")
+    _i32(ids, T, "token ids")
+    out = torch.empty((T, width), dtype=out_dtype, device=z.device)
+    _check(lib().gs_side_gate(_p(z), _dt(z), z.shape[1], _p(table), _dt(table), table.shape[1], offset, _p(ids), dim, _p(out),
+                              _dt(out), width, T, _stream()))
+    return out

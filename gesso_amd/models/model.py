@@ -13,7 +13,7 @@ import torch
 
 from ..config.spec import ModelSpec
 from ..errors import ConfigError
-from ..parts.base import MATRIX, TABLE, VECTOR, TensorSpec
+from ..parts.base import MATRIX, TABLE, VECTOR, PagedKV, TensorSpec
 from ..parts.registry import build, part_class
 from ..parts.rmsnorm import ResidualStream, row_weight_of
 
@@ -54,6 +54,24 @@ def tied_aliases(spec: ModelSpec) -> Dict[str, str]:
     return {}
 
 
+def schedule_cache_needs(spec: ModelSpec) -> List[Optional[object]]:
+    """See :meth:`Model.cache_needs`."""
+    out: List[Optional[object]] = []
+    for call in spec.schedule:
+        b = spec.blocks[call.layer]
+        need = part_class("block", b).cache_need(b)
+        if call.cache is None:
+            out.append(need)
+            continue
+        src = call.cache
+        while spec.schedule[src].cache is not None:
+            src = spec.schedule[src].cache
+        if isinstance(need, PagedKV) and isinstance(out[src], PagedKV):
+            out[src] = out[src].reaching(need)
+        out.append(None)
+    return out
+
+
 class Model:
     def __init__(self, spec: ModelSpec, rt):
         self.spec = spec
@@ -66,13 +84,9 @@ class Model:
         self.reentry_weight = self.reentry_step = None
 
     def cache_needs(self) -> List[Optional[object]]:
-        """For each entry of the schedule: what its own cache must hold (None: none, or it reads another's)."""
-        out = []
-        for call in self.spec.schedule:
-            b = self.spec.blocks[call.layer]
-            need = part_class("block", b).cache_need(b)
-            out.append(None if call.cache is not None else need)
-        return out
+        """For each entry of the schedule: what its own cache must hold (None: none, or it reads another's).  A cache that
+        later calls read keeps the rows that any of its readers may still see."""
+        return schedule_cache_needs(self.spec)
 
     def bind(self, tensors: Dict[str, torch.Tensor]) -> None:
         s = self.spec

@@ -9,7 +9,9 @@ Interfaces (duck-typed; the classes below are convenient bases):
 
 * norm            ``tensor_specs(spec)``, ``bind(tensors)``, ``add_norm(stream, rows=None, out=None) -> normed``;
                   optional hint ``row_weight``: a float32 vector ``w`` with ``norm(x) = inv_rms(x) * (x * w)``, which
-                  lets whatever writes the stream before the norm leave the rows pre-weighted (None: no such form)
+                  lets whatever writes the stream before the norm leave the rows pre-weighted (None: no such form);
+                  optional ``seam()``: the norm in the form that the kernel between two sub-layers takes
+                  (``ops.SeamNorm``), for blocks that norm a sub-layer's output as well
 * position        ``tensor_specs(spec)`` (usually none), ``bind``, attributes
                   ``cos``, ``sin`` (``(max_position, rotary_dim/2)`` float32), ``rotary_dim`` and ``layout``
                   (``"half"``: pairs ``(i, i + rotary_dim/2)``, ``"interleaved"``: ``(2i, 2i + 1)``);
@@ -18,6 +20,7 @@ Interfaces (duck-typed; the classes below are convenient bases):
                   (a mixer made of several, each with a cache of its own: ``cache`` is then a tuple of views),
                   ``bind(tensors)``, ``forward(x, ctx, cache) -> (T, hidden)``
 * feed-forward    ``tensor_specs(spec)``, ``bind(tensors)``, ``forward(x, ctx) -> (T, hidden)``
+* side input      the same, with ``out_seam()``: the norm its output passes before it is added (a form the seam kernel takes)
 * block           ``tensor_specs(spec)``, ``cache_need(spec)``, ``bind``,
                   ``forward(stream, ctx, cache)`` on a :class:`ResidualStream`; optional hint ``first_norm``: the
                   norm that reads the stream first when the block runs (None: unknown)
@@ -26,7 +29,7 @@ Interfaces (duck-typed; the classes below are convenient bases):
 """
 from __future__ import annotations
 
-from dataclasses import dataclass
+from dataclasses import dataclass, replace
 from typing import Dict, Optional, Tuple
 
 MATRIX = "matrix"     # operand of a matrix product: keeps the stored width (bfloat16 stays bfloat16)
@@ -67,6 +70,17 @@ class PagedKV:
     def pages_kept(self, page_size: int) -> int:
         """How many pages at a sequence's start hold positions that stay readable whatever has passed."""
         return -(-int(self.keep_first) // page_size) if self.window is not None and self.chunk is None else 0
+
+    def reaching(self, other: "PagedKV") -> "PagedKV":
+        """What a cache must keep so that ``other``'s reader, too, finds every row it may see: the rows' shape is this
+        cache's (``other`` must agree), the reach the wider of the two."""
+        if (self.n_kv_heads, self.head_dim, self.value_width) != (other.n_kv_heads, other.head_dim, other.value_width):
+            raise ValueError(f"a reader of rows {other} cannot share a cache of {self}")
+        if self.chunk != other.chunk:
+            raise ValueError("readers of one cache cut their positions into the same runs, or none does")
+        window = None if self.window is None or other.window is None else max(self.window, other.window)
+        keep = max(self.keep_first, other.keep_first) if window is not None else 0
+        return replace(self, window=window, keep_first=keep)
 
     def first_needed(self, length: int) -> int:
         """The oldest position that the token after ``length`` cached ones can read."""

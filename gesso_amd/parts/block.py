@@ -117,6 +117,97 @@ class OutNormBlock(PreNormBlock):
         return False
 
 
+class SandwichBlock(Part):
+    """``h += mult * norm_b(mixer(norm_a(h)))``, ``h += mult * norm_d(ffn(norm_c(h)))``, ``h += mult * norm_s(side(h))``: a
+    norm before and after every sub-layer, and at the end what the token brings to this layer by itself.  Between two
+    sub-layers one kernel norms the one's output, adds it to the stream and norms the stream for the other
+    (``ops.norm_seam``); the rows for whoever reads the stream after the block are made in the last of them."""
+
+    ROLES = (("mixer_norm", "norm"), ("mixer", "mixer"), ("mixer_out_norm", "norm"), ("ffn_norm", "norm"), ("ffn", "ffn"),
+             ("ffn_out_norm", "norm"), ("side", "side"))
+
+    @staticmethod
+    def _parts(spec):
+        for role, category in SandwichBlock.ROLES:
+            if role.startswith("ffn") and spec.ffn is None:
+                continue
+            sub = getattr(spec, role)
+            if sub is not None:
+                yield role, category, sub
+
+    def __init__(self, spec, rt):
+        super().__init__(spec, rt)
+        self.ffn = self.side = None
+        for role, category, sub in self._parts(spec):
+            part = build(category, sub, rt)
+            if category == "norm" and not hasattr(part, "seam"):
+                raise ValueError(f"a norm of kind {sub.kind!r} has no form for the pass between two sub-layers")
+            setattr(self, role, part)
+
+    @staticmethod
+    def tensor_specs(spec):
+        return {f"{role}.{name}": ts for role, category, sub in SandwichBlock._parts(spec)
+                for name, ts in part_class(category, sub).tensor_specs(sub).items()}
+
+    @staticmethod
+    def cache_need(spec):
+        cls = part_class("mixer", spec.mixer)
+        return cls.cache_need(spec.mixer) if hasattr(cls, "cache_need") else None
+
+    def bind(self, tensors):
+        for role, _, _ in self._parts(self.spec):
+            getattr(self, role).bind(sub_tensors(tensors, role))
+
+    @property
+    def first_norm(self):
+        return self.mixer_norm
+
+    def forward(self, stream, ctx, cache):
+        rt, ops, s = self.rt, self.rt.ops, self.spec
+        after = stream.following if hasattr(stream.following, "seam") else None
+        with rt.stage("norm"):
+            x = rt.dense(self.mixer_norm.add_norm(stream))
+        stream.flush(rt)
+        stream.pending = stream.ssq = stream.xs = stream.xs_for = stream.normed = stream.rows = None
+
+        def seam(y, post, pre):
+            """``pre``: the norm that reads the stream next, "raw" (the stream itself), or None (nobody here)."""
+            if pre is None:
+                return ops.norm_seam(stream.res, y, post, s.mult, None)
+            if pre == "raw":
+                if rt.dtype == stream.res.dtype:
+                    ops.norm_seam(stream.res, y, post, s.mult, None)
+                    return stream.res
+                return ops.norm_seam(stream.res, y, post, s.mult, None, rt.dtype)
+            return ops.norm_seam(stream.res, y, post, s.mult, pre.seam(), rt.dtype)
+
+        end = "raw" if self.side is not None else after
+        with rt.stage(getattr(self.mixer, "stage", "mixer")):
+            # (the last product is not deferred into the stream: its rows pass a norm first)
+            kw = {"out_dtype": rt.dtype} if getattr(self.mixer, "takes_out_dtype", False) else {}
+            y = rt.dense(self.mixer.forward(x, ctx, cache, **kw))
+        with rt.stage("norm"):
+            x = seam(y, self.mixer_out_norm.seam(), self.ffn_norm if self.ffn is not None else end)
+        if self.ffn is not None:
+            with rt.stage(getattr(self.ffn, "stage", "ffn")):
+                y = rt.dense(self.ffn.forward(x, ctx))
+            with rt.stage("norm"):
+                x = seam(y, self.ffn_out_norm.seam(), end)
+        if self.side is not None:
+            with rt.stage("side"):
+                y = self.side.forward(x, ctx)
+            with rt.stage("norm"):
+                x = seam(y, self.side.out_seam(), after)
+        if after is not None:
+            stream.normed, stream.xs_for = x, after
+
+    @property
+    def graph_safe(self) -> bool:
+        return all(getattr(getattr(self, role), "graph_safe", False) for role, _, _ in self._parts(self.spec))
+
+    portions_recordable = False
+
+
 class ParallelBlock(PreNormBlock):
     """``h += mixer(norm_a(h)) + ffn(norm_b(h))``: both sub-layers read the stream as it enters the block, each
     through its own norm.  One kernel adds what the block before left (its two results) and norms the row for both
@@ -243,5 +334,6 @@ class SharedNormBlock(Part):
 
 register("block", "prenorm", PreNormBlock)
 register("block", "shared_norm", SharedNormBlock)
+register("block", "sandwich", SandwichBlock)
 register("block", "parallel", ParallelBlock)
 register("block", "outnorm", OutNormBlock)

@@ -1,6 +1,6 @@
 """Recurrent mixers whose matrix state fades by a factor that depends on the token.
 
-Both keep, per head, a state ``S`` (``key_dim x value_dim``, float32 in both precisions, zero at a request's start) in the
+All keep, per head, a state ``S`` (``key_dim x value_dim``, float32 in both precisions, zero at a request's start) in the
 request's slot and advance it token by token with one kernel (``ops.gated_state_scan``), whose sums run in one order
 whatever the step's cut.  A step that brings a portion of ``2 * SEGMENT`` tokens or more walks its portions in segments
 side by side (over a segment the state goes ``S -> M S + B``; ``ops.gated_state_scan_segments``); results then differ
@@ -26,6 +26,16 @@ the two bottlenecks side by side, with zeros where one's features meet the other
     [q | k | v | z] = W_in x,   alpha = sigmoid(W_up (W_down x) + b)^(1/tau)           n_heads x key_dim decays
     S <- diag(alpha) S + k v^T;  o = S^T (q key_dim^-0.5)
     out = W_o (rms(o) * w * silu(z))
+
+``MatrixMemory`` (a matrix memory with exponential gates):
+
+    [q | k | v | z] = W_in x,   [a | b] = W_gates x (float32 sums)
+    i = cap tanh((a + b_i) / cap),   f = log sigmoid(cap tanh((b + b_f) / cap));   p <- max(f + p, i)       per head
+    S <- exp(f + p_before - p) S + exp(i - p) k [v | 1]^T;   [o | d] = S^T (q key_dim^-0.5)
+    out = W_o (rms(o / (max(|d|, exp(-p)) + 1e-6)) * w * sigmoid(z))
+
+The sum of the keys that the output is divided by is the state's last column, whose values are ones; the running maximum
+``p`` lies in the request's slot beside the state.
 
 From the convolutions' outputs (or the input product) to the gated norm nothing is rounded to the activation type:
 unit norms, gates, decays and the state are float32.
@@ -212,5 +222,57 @@ class GatedLinear(Part):
         return rt.linear(y, self.w_out, out_dtype=out_dtype)
 
 
+class MatrixMemory(Part):
+    graph_safe = True
+    stage, out_stage = "memory_mixer", "memory_out"
+
+    def __init__(self, spec, rt):
+        super().__init__(spec, rt)
+        if spec.key_dim > rt.ops.GATED_STATE_MAX_KEY:
+            raise ValueError(f"keys of {spec.key_dim} features: the state kernel holds up to {rt.ops.GATED_STATE_MAX_KEY}")
+        if not spec.gate_cap > 0:
+            raise ValueError("gate_cap must be positive")
+
+    @staticmethod
+    def tensor_specs(spec):
+        W, H, n, m = spec.hidden, spec.n_heads, spec.key_dim, spec.value_dim
+        return {"q_proj.weight": TensorSpec((H * n, W), MATRIX), "k_proj.weight": TensorSpec((H * n, W), MATRIX),
+                "v_proj.weight": TensorSpec((H * m, W), MATRIX), "gate_proj.weight": TensorSpec((H * m, W), MATRIX),
+                "input_gate.weight": TensorSpec((H, W), MATRIX), "input_gate.bias": TensorSpec((H,), VECTOR),
+                "forget_gate.weight": TensorSpec((H, W), MATRIX), "forget_gate.bias": TensorSpec((H,), VECTOR),
+                "out_norm.weight": TensorSpec((H * m,), VECTOR, "one_plus_normal"), "out_proj.weight": TensorSpec((W, H * m), MATRIX)}
+
+    @staticmethod
+    def cache_need(spec):
+        return SlotState((("state", (spec.n_heads, spec.key_dim, spec.value_dim + 1), "float32"),
+                          ("peak", (spec.n_heads,), "float32")))
+
+    def bind(self, tensors):
+        rt = self.rt
+        self.w_in = rt.prepare(stacked([tensors[k + "_proj.weight"] for k in ("q", "k", "v", "gate")]))
+        self.w_gates = rt.prepare(stacked([tensors["input_gate.weight"], tensors["forget_gate.weight"]]))
+        self.b_i, self.b_f = tensors["input_gate.bias"], tensors["forget_gate.bias"]
+        self.w_out = rt.prepare(tensors["out_proj.weight"])
+        self.norm_weight = tensors["out_norm.weight"]
+
+    takes_out_dtype = True
+
+    def forward(self, x, ctx, cache, out_dtype=None):
+        s, rt, ops = self.spec, self.rt, self.rt.ops
+        H, n, m = s.n_heads, s.key_dim, s.value_dim
+        x = rt.dense(x)
+        with rt.stage("memory_in"):
+            rows = rt.linear(x, self.w_in)                             # q | k | v | z (| spare columns)
+            gates = ops.exp_gates(rt.narrow_linear(x, self.w_gates), 0, H, self.b_i, self.b_f, s.gate_cap, cache.state["peak"],
+                                  ctx.q_start, ctx.slots, ctx.nseq, H)
+        with rt.stage("memory_state"):
+            o = _scan(ops, ctx, (rows, 0, H * n, 2 * H * n, H, H, n, m + 1, gates, 0, False), cache.state["state"],
+                      q_scale=float(n) ** -0.5, beta=gates, ob=H, delta=False, ones=True)
+        with rt.stage("memory_norm"):
+            y = ops.memory_outnorm(o, gates, rows, 2 * H * n + H * m, self.norm_weight, s.eps, H, m, rt.dtype)
+        return rt.linear(y, self.w_out, out_dtype=out_dtype)
+
+
+register("mixer", "matrix_memory", MatrixMemory)
 register("mixer", "gated_delta", GatedDelta)
 register("mixer", "gated_linear", GatedLinear)

@@ -17,11 +17,16 @@ attends over the cached rows themselves, and because the softmax weights sum ove
 so a position's result does not depend on how its sequence was cut.
 
 ``W_dq``, ``W_dkv`` and ``W_g`` read the same input and are laid side by side at load: one product.
+
+With ``sinks`` the softmax's denominator has one more term ``exp(s_h)`` without a row.  A mixer with ``own_rows = False`` has
+no ``W_dkv``: it attends over the rows that an earlier call of the schedule has written, by its own window, which may reach
+further back than that call's (the cache keeps what the widest reader sees).
 """
 from __future__ import annotations
 
 import torch
 
+from ..errors import InvalidPlan
 from .base import MATRIX, VECTOR, PagedKV, Part, TensorSpec
 from .registry import build, register
 
@@ -55,9 +60,14 @@ class LatentAttention(Part):
     def tensor_specs(spec):
         W, H, n, r, dv, qr, c = spec.hidden, spec.n_heads, spec.plain_dim, spec.rot_dim, spec.value_dim, spec.q_rank, spec.kv_rank
         out = {"q_down.weight": TensorSpec((qr, W), MATRIX), "q_norm.weight": TensorSpec((qr,), VECTOR, "one_plus_normal"),
-               "q_up.weight": TensorSpec((H * (n + r), qr), MATRIX), "kv_down.weight": TensorSpec((c + r, W), MATRIX),
-               "kv_norm.weight": TensorSpec((c,), VECTOR, "one_plus_normal"), "k_up.weight": TensorSpec((H * n, c), MATRIX),
-               "v_up.weight": TensorSpec((H * dv, c), MATRIX), "out.weight": TensorSpec((W, H * dv), MATRIX)}
+               "q_up.weight": TensorSpec((H * (n + r), qr), MATRIX)}
+        if getattr(spec, "own_rows", True):
+            out.update({"kv_down.weight": TensorSpec((c + r, W), MATRIX),
+                        "kv_norm.weight": TensorSpec((c,), VECTOR, "one_plus_normal")})
+        out.update({"k_up.weight": TensorSpec((H * n, c), MATRIX), "v_up.weight": TensorSpec((H * dv, c), MATRIX),
+                    "out.weight": TensorSpec((W, H * dv), MATRIX)})
+        if getattr(spec, "sinks", False):
+            out["sinks"] = TensorSpec((H,), VECTOR)
         if spec.gated:
             out["gate.weight"] = TensorSpec((H * dv if getattr(spec, "gate_each", False) else H, W), MATRIX)
         return out
@@ -69,18 +79,21 @@ class LatentAttention(Part):
     def bind(self, tensors):
         s, rt = self.spec, self.rt
         H, n, r, dv, c = s.n_heads, s.plain_dim, s.rot_dim, s.value_dim, s.kv_rank
-        w_dkv, w_uq = tensors["kv_down.weight"], tensors["q_up.weight"]
+        w_dkv, w_uq = tensors.get("kv_down.weight"), tensors["q_up.weight"]
         if self.reorder:
-            order = torch.cat([torch.arange(0, r, 2), torch.arange(1, r, 2)]).to(w_dkv.device)
-            w_dkv = torch.cat([w_dkv[:c], w_dkv[c:][order]], 0)
+            order = torch.cat([torch.arange(0, r, 2), torch.arange(1, r, 2)]).to(w_uq.device)
+            if w_dkv is not None:
+                w_dkv = torch.cat([w_dkv[:c], w_dkv[c:][order]], 0)
             per_head = torch.cat([torch.arange(n, device=order.device), n + order])
             rows = (torch.arange(H, device=order.device)[:, None] * (n + r) + per_head[None, :]).reshape(-1)
             w_uq = w_uq[rows].contiguous()
-        ws = [tensors["q_down.weight"], w_dkv] + ([tensors["gate.weight"]] if s.gated else [])
+        ws = [tensors["q_down.weight"]] + ([w_dkv] if w_dkv is not None else []) + ([tensors["gate.weight"]] if s.gated else [])
+        self.gate_at = s.q_rank + (c + r if w_dkv is not None else 0)
+        self.sinks = tensors.get("sinks")
         if len({w.dtype for w in ws}) > 1:
             ws = [w.float() for w in ws]
         self.w_in = rt.prepare(_pad_rows(torch.cat(ws, 0)))
-        self.q_norm, self.kv_norm = tensors["q_norm.weight"], tensors["kv_norm.weight"]
+        self.q_norm, self.kv_norm = tensors["q_norm.weight"], tensors.get("kv_norm.weight")
         self.w_uq = rt.prepare(w_uq)
         # W_uk[h]^T as the weight of a per-head product: (H, c, n); W_uv[h]: (H, dv, c)
         self.uk_t = tensors["k_up.weight"].reshape(H, n, c).transpose(1, 2).contiguous() if n else None
@@ -93,6 +106,8 @@ class LatentAttention(Part):
         x = rt.dense(x)
         T = x.shape[0]
         with rt.stage("attn_proj"):
+            if self.kv_norm is None and cache.write:
+                raise InvalidPlan("a mixer without latent rows of its own must read another call's cache")
             down = rt.linear(x, self.w_in)                     # [query latent | kv latent | shared rotated key | gate]
             a = ops.latent_prep(down, 0, qr, qr, c, r, self.q_norm, self.kv_norm, s.eps, pos.cos, pos.sin, ctx.positions,
                                 ctx.seq_of_token, cache.block_table, cache.page_size, cache.k, write_kv=cache.write)
@@ -104,7 +119,7 @@ class LatentAttention(Part):
         with rt.stage("attn_core"):
             mixed = self.attend(qa, ctx, cache)
         o = torch.empty((T, H * dv), dtype=mixed.dtype, device=mixed.device)
-        ops.heads_product(mixed, c, self.uv, o, dv, c, gate=down[:, qr + c + r:] if s.gated else None,
+        ops.heads_product(mixed, c, self.uv, o, dv, c, gate=down[:, self.gate_at:] if s.gated else None,
                           gate_each=bool(s.gated and getattr(s, "gate_each", False)))
         return rt.linear(o, self.w_out)
 
@@ -127,9 +142,10 @@ class LatentAttention(Part):
                 blocks = ctx.T * -(-s.n_heads // 64)
                 nsplit = max(1, min(longest // 64, 64, self.rt.compute_units // max(1, blocks)))
             return ops.attention_latent_mfma(qa, cache.k, ctx.positions, tiles, cache.block_table, cache.page_size,
-                                             s.window, s.scale, s.n_heads, s.kv_rank, s.rot_dim, ctx.T, nsplit=nsplit)
+                                             s.window, s.scale, s.n_heads, s.kv_rank, s.rot_dim, ctx.T, nsplit=nsplit,
+                                             sinks=self.sinks)
         return ops.attention_latent(qa, cache.k, ctx.positions, ctx.seq_of_token, cache.block_table, cache.page_size,
-                                    s.window, s.scale, s.n_heads, s.kv_rank, s.rot_dim, ctx.T)
+                                    s.window, s.scale, s.n_heads, s.kv_rank, s.rot_dim, ctx.T, sinks=self.sinks)
 
 
 register("mixer", "latent_attention", LatentAttention)

@@ -1,5 +1,5 @@
-"""An ungated feed-forward: ``W_down act(W_up x)``, no biases; ``act`` is the error-function or tanh form of gelu, or silu,
-applied in float32 to the product's rows."""
+"""An ungated feed-forward: ``W_down act(W_up x)``, no biases; ``act`` is the error-function or tanh form of gelu, silu or
+the square of relu, applied in float32 to the product's rows."""
 from __future__ import annotations
 
 from .base import MATRIX, Part, TensorSpec

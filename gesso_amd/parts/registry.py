@@ -1,4 +1,4 @@
-"""Registries of part kinds: mixers, feed-forwards, norms, position encodings, blocks.
+"""Registries of part kinds: mixers, feed-forwards, norms, position encodings, blocks, side inputs.
 
 A spec's ``kind`` picks the class.  Registering a new kind (from a test, from another
 architecture's file) needs no change here: ``register("mixer", "my_kind", MyMixer)``.
@@ -9,7 +9,7 @@ from typing import Dict
 
 from ..errors import ConfigError
 
-CATEGORIES = ("mixer", "ffn", "norm", "position", "block")
+CATEGORIES = ("mixer", "ffn", "norm", "position", "block", "side")
 _PARTS: Dict[str, Dict[str, type]] = {c: {} for c in CATEGORIES}
 
 

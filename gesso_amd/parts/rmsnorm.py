@@ -131,6 +131,10 @@ class RMSNorm(Part):
         return y
 
 
+    def seam(self):
+        return self.rt.ops.SeamNorm("rms", self.weight, eps=self.spec.eps)
+
+
 class GroupRMSNorm(Part):
     """RMS norm in parts: the row is cut into ``groups`` equal consecutive parts, each divided by its own
     ``sqrt(mean(part^2) + eps)``; then the weight.  One part: the plain norm.  float32 arithmetic."""
@@ -192,6 +196,42 @@ class LayerNorm(Part):
         return y
 
 
+class DynTanh(Part):
+    """``tanh(alpha x) w + b``: no mean, no variance, so the pass is elementwise.  float32 arithmetic.  Between two
+    sub-layers a block asks for :meth:`seam` and lets one kernel do this norm and the add before it."""
+
+    graph_safe = True
+
+    @staticmethod
+    def tensor_specs(spec):
+        return {"weight": TensorSpec((spec.size,), VECTOR, "one_plus_normal"), "bias": TensorSpec((spec.size,), VECTOR),
+                "alpha": TensorSpec((), VECTOR, "one_plus_normal")}
+
+    def bind(self, tensors):
+        self.weight, self.bias = tensors["weight"], tensors["bias"]
+        self.alpha = tensors["alpha"].reshape(1).contiguous()
+        self._seam = self.rt.ops.SeamNorm("dyn_tanh", self.weight, self.bias, self.alpha)
+
+    def seam(self):
+        return self._seam
+
+    def add_norm(self, stream: ResidualStream, rows=None, out=None, out_dtype=None):
+        """Add what is pending to the stream, then norm it (only ``rows`` of it when given); rows that the last writer
+        of the stream made for this norm are taken as they are."""
+        rt = self.rt
+        dtype = out_dtype or rt.dtype
+        if rows is None and out is None and stream.xs_for is self and stream.normed is not None and stream.normed.dtype == dtype:
+            return stream.normed
+        if isinstance(stream.pending, tuple) or stream.bias is not None or rows is not None:
+            stream.flush(rt)
+        y = rt.ops.norm_seam(stream.res, stream.pending, None, 1.0, self._seam, dtype, rows=rows, out=out)
+        if stream.pending is not None:
+            stream.pending = None
+            stream.ssq = stream.xs = stream.xs_for = stream.normed = stream.rows = None
+        return y
+
+
 register("norm", "rmsnorm", RMSNorm)
+register("norm", "dyn_tanh", DynTanh)
 register("norm", "layernorm", LayerNorm)
 register("norm", "group_rmsnorm", GroupRMSNorm)

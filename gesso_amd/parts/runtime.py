@@ -208,6 +208,14 @@ class Runtime:
                 return ops.gemm_mfma(x, w, out_dtype=out_dtype, out=out)
         return ops.gemm_tiled(x, w, bias, out_dtype=out_dtype, out=out)
 
+    def narrow_linear(self, x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+        """``x @ w.T`` in float32 for a weight of few rows (the gates of a few heads, a bottleneck): for more rows than the
+        weight-streaming kernel takes, by the kernel that shares K out between a block's wavefronts."""
+        ops = self.ops
+        if not ops.skinny_ok(x, w) and ops.narrow_ok(x, w):
+            return ops.gemm_narrow(x, w, torch.float32)
+        return self.linear(x, w, out_dtype=torch.float32)
+
     LIBRARY_WORKSPACE = 64 << 20
 
     def _library_product(self, x, w, out):
