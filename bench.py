@@ -63,6 +63,10 @@ def weight_bytes(engine) -> int:
     for b in m.blocks:
         for part in (getattr(b, name, None) for name in ("mixer_norm", "norm", "mixer", "ffn_norm", "ffn")):
             tensors += of(part)
+        for part in (getattr(b, name, None) for name in ("mixer_out_norm", "ffn_out_norm")):
+            tensors += of(part)
+        if getattr(b, "side", None) is not None:       # (of a side input's table a step reads its tokens' rows only)
+            tensors += [b.side.w_gate, b.side.w_proj]
         tensors += [v for v in vars(b).values() if isinstance(v, torch.Tensor)]      # a block's own (an input convolution's taps)
     for t in tensors:
         if t.data_ptr() not in seen:
@@ -613,6 +617,66 @@ def bilolix_workload(steps: int = 64, warmup: int = 8, sizes=("1024", "2048"), o
     return out
 
 
+VAKESUN_SIZES = {
+    # eight layers: attention, matrix memory, attention, latent attention, and the same four again, the second latent
+    # layer over the first one's rows; attention and latent layers have a feed-forward, the memories none.  Widths 1,024
+    # and 2,048 have the latent mixer of Makuzen's sizes (beside which they are measured: it is the model with the same
+    # embedding scale, residual factor, output norms and latent rows) and the state of Kuditar's linear attention (the
+    # model with the same state kernel); width 1,536 has heads of 96
+    "1024": dict(width=1024, attn=(16, 4, 64, 32), memory=(8, 64, 128), latent=(16, 64, 64, 384, 256), window=1024, ff=6912, side=128,
+                 vocab=65536, beside=("makuzen", "kuditar")),
+    "2048": dict(width=2048, attn=(16, 4, 128, 64), memory=(16, 64, 128), latent=(16, 128, 128, 768, 512), window=2048, ff=12288,
+                 side=256, vocab=65536, beside=("makuzen", "kuditar")),
+    "1536": dict(width=1536, attn=(16, 4, 96, 48), memory=(8, 128, 256), latent=(16, 96, 96, 512, 384), window=1024, ff=9216, side=192,
+                 vocab=65536, beside=()),
+}
+
+
+def vakesun_config(size: str, max_position: int = 4096):
+    from gesso_amd.config import (GroupedAttentionConfig, MatrixMemoryConfig, SinkLatentConfig, SquaredReluConfig, VakesunConfig,
+                                  VakesunLayer, YarnScaling, YarnTurn)
+    z = VAKESUN_SIZES[size]
+    h, g, d, turned = z["attn"]
+    attn = VakesunLayer("attention", GroupedAttentionConfig(h, g, d, d, d ** -0.5, YarnTurn(5e5, turned, YarnScaling(4.0, 1024.0, 32.0, 1.0))),
+                        SquaredReluConfig(z["ff"]))
+    memory = VakesunLayer("mlstm", MatrixMemoryConfig(*z["memory"], 15.0), None)
+    lh, ld, lvd, qr, kr = z["latent"]
+    latent = [VakesunLayer("latent_attention", SinkLatentConfig(lh, ld, lvd, ld ** -0.5, qr, kr, z["window"], src), SquaredReluConfig(z["ff"]))
+              for src in (None, 3)]
+    return VakesunConfig(vocab=z["vocab"], width=z["width"], layers=(attn, memory, attn, latent[0], attn, memory, attn, latent[1]),
+                         embedding_scale=12.0, norm_eps=1e-6, residual_mult=0.7, side_dim=z["side"], max_position=max_position)
+
+
+def vakesun_workload(steps: int = 64, warmup: int = 8, sizes=("1024", "2048", "1536"), only: str = "", batches=(8, 64)) -> dict:
+    """Vakesun (elementwise norms on both sides of every sub-layer, softmax attention, matrix memories with exponential
+    gates, latent attention with sinks, a token's own input to every layer) at three sets of layer sizes, beside Makuzen
+    and Kuditar of the same width and depth: a 2,048-token prompt in one step, and decode steps at 512-token prompts."""
+    from gesso_amd import Engine
+    from gesso_amd.parts import RuntimeOptions
+    out = {"metric": "Vakesun beside Makuzen and Kuditar at equal width and depth: prefill and decode tok/s", "unit": "tok/s", "dtype": "bf16",
+           "data": "synthetic: uniform random token ids, random weights N(0, 0.02)", "sizes": {}}
+    others = {"makuzen": makuzen_config, "kuditar": kuditar_config}
+    for size in sizes:
+        row = {}
+        for name, cfg in [("vakesun", vakesun_config(size))] + [(n, others[n](size)) for n in VAKESUN_SIZES[size]["beside"]]:
+            if only and only != name:
+                continue
+            engine = Engine.from_config(cfg, seed=0, dtype="bfloat16", page_size=16, max_context=4096,
+                                        max_tokens=max(batches) * (512 + steps + warmup + 32) + 4096, num_slots=max(batches) + 1,
+                                        options=RuntimeOptions(tune_library=True))
+            sec = prefill_run(engine, cfg, 2048)
+            r = {"prefill_tok_s": round(2048 / sec, 1), "prefill_ms": round(sec * 1e3, 3), "weights_gb": round(weight_bytes(engine) / 1e9, 3)}
+            for b in batches:
+                dt, _ = decode_run(engine, cfg, b, 512, steps, warmup, seed=40 + b)
+                r[f"decode_b{b}_tok_s"] = round(b * steps / dt, 1)
+                r[f"decode_b{b}_ms"] = round(dt / steps * 1e3, 4)
+            row[name] = r
+            del engine
+            torch.cuda.empty_cache()
+        out["sizes"][size] = row
+    return out
+
+
 def main() -> int:
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -632,7 +696,7 @@ def main() -> int:
     ap.add_argument("--launched-portions", action="store_true", help="launch the steps with prompt portions kernel by kernel instead of "
                     "replaying recordings of them (the prefill of the default line, --workload serve)")
     ap.add_argument("--token-budget", type=int, default=4096, help="--workload serve: the most tokens a step holds")
-    ap.add_argument("--workload", default="decode", choices=["decode", "serve", "long", "gemm", "stages", "makuzen", "fazezen", "togalorn", "kuditar", "bilolix"],
+    ap.add_argument("--workload", default="decode", choices=["decode", "serve", "long", "gemm", "stages", "makuzen", "fazezen", "togalorn", "kuditar", "bilolix", "vakesun"],
                     help="decode: the default line; serve: continuous batching at LFM2-350M sizes; long: LFM2-2.6B "
                          "sizes at a context of 32,768; gemm: the products of a 2,048-token prompt, ours beside the vendor's; "
                          "stages: the decode step stage by stage; makuzen: the Makuzen design at two sets of layer sizes "
@@ -645,6 +709,8 @@ def main() -> int:
     ap.add_argument("--kuditar-only", default="", choices=["", "kuditar", "fazezen"], help="--workload kuditar: one of the two models (for profiling)")
     ap.add_argument("--bilolix-sizes", default="1024,2048", help="--workload bilolix: which of its sizes")
     ap.add_argument("--bilolix-only", default="", choices=["", "bilolix", "kuditar"], help="--workload bilolix: one of the two models (for profiling)")
+    ap.add_argument("--vakesun-sizes", default="1024,2048,1536", help="--workload vakesun: which of its sizes")
+    ap.add_argument("--vakesun-only", default="", choices=["", "vakesun", "makuzen", "kuditar"], help="--workload vakesun: one of the three models (for profiling)")
     ap.add_argument("--makuzen-sizes", default="1024,2048", help="--workload makuzen: which of its sizes")
     ap.add_argument("--makuzen-only", default="", choices=["", "makuzen", "lfm2"], help="--workload makuzen: one of the two models (for profiling)")
     args = ap.parse_args()
@@ -670,6 +736,10 @@ def main() -> int:
         if args.workload == "bilolix":
             print(json.dumps(bilolix_workload(min(args.steps, 64), min(args.warmup, 8), tuple(args.bilolix_sizes.split(",")),
                                               args.bilolix_only)))
+            return 0
+        if args.workload == "vakesun":
+            print(json.dumps(vakesun_workload(min(args.steps, 64), min(args.warmup, 8), tuple(args.vakesun_sizes.split(",")),
+                                              args.vakesun_only)))
             return 0
         if args.workload == "togalorn":
             print(json.dumps(togalorn_workload(min(args.steps, 64), min(args.warmup, 8), tuple(args.togalorn_sizes.split(",")),

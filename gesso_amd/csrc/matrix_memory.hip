@@ -7,32 +7,41 @@
 //   gates[t, h] = exp(f + p_(t-1) - p_t)                 what the memory keeps
 //   gates[t, H + h] = exp(i - p_t)                       with what the token is written
 //   gates[t, 2 H + h] = exp(-p_t)                        the least the output is divided by
-// A wavefront per (sequence, head), 64 tokens a turn: a token takes the maximum from p to max(p + f, i), and such maps
-// compose, (f1, i1) then (f2, i2) = (f1 + f2, max(i1 + f2, i2)), so six steps between lanes give every token's p.
+// With `logs` the first two are their base-2 logarithms instead.  A token takes the maximum from p to max(p + f, i), and such
+// maps compose, (f1, i1) then (f2, i2) = (f1 + f2, max(i1 + f2, i2)), so six steps between lanes give 64 tokens' p.  Steps of
+// few tokens: a wavefront per (sequence, head), four heads a block.  Longer portions: a block per (sequence, head), whose
+// wavefronts take 64 tokens each and hand their maps on through LDS.
 //
-// memory_outnorm: o (T, H (m + 1)) float32, a head's m columns and then the column whose values are ones (n . q):
+// memory_outnorm: a head's m columns o and the number n . q (`den`), float32:
 //   u = o / (max(|n . q|, exp(-p)) + 1e-6);   out = u / sqrt(mean(u^2) + eps) * w * sigmoid(gate)      per head
+// Head h of token t has its columns at o[(t H + h) hs] and its number at den[(t H + h) ds].
 #include "common.h"
 
-__global__ void __launch_bounds__(256)
+#define MM_LOG2E 1.4426950408889634f
+
+// W wavefronts share a (sequence, head); W = 1: each of the block's four has a head of its own.
+template <int W>
+__global__ void __launch_bounds__(W == 1 ? 256 : W * 64)
 exp_gates_kernel(const float* __restrict__ z, int ldz, int oi, int of, const float* __restrict__ bi,
                  const float* __restrict__ bf, float cap, float* __restrict__ peak, const int* __restrict__ q_start,
-                 const int* __restrict__ slots, float* __restrict__ gates, int H) {
-  const int lane = threadIdx.x & 63, h = blockIdx.y * 4 + (threadIdx.x >> 6), seq = blockIdx.x;
-  if (h >= H) return;
+                 const int* __restrict__ slots, float* __restrict__ gates, int H, int logs) {
+  __shared__ float wf[W], wi[W];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, seq = blockIdx.x;
+  const int h = W == 1 ? blockIdx.y * 4 + wave : blockIdx.y;
+  if (h >= H) return;                                // (with W > 1 there is a block per head: all of it or nothing)
   const int t0 = q_start[seq], t1 = q_start[seq + 1];
   if (t1 <= t0) return;
   float* own = peak + (size_t)slots[seq] * H + h;
   float p = *own;
-  const float b_i = bi[h], b_f = bf[h];
-  for (int tb = t0; tb < t1; tb += 64) {
-    const int t = tb + lane;
-    const bool live = t < t1;
+  const float b_i = bi[h], b_f = bf[h], inv_cap = 1.0f / cap;
+  for (int tb = t0; tb < t1; tb += 64 * W) {
+    const int t = tb + (W == 1 ? lane : (int)threadIdx.x);
+    const bool in = t < t1;
     float f = 0.f, i = -INFINITY;                    // (a lane without a token: the map that changes nothing)
-    if (live) {
+    if (in) {
       const float zi = z[(size_t)t * ldz + oi + h] + b_i, zf = z[(size_t)t * ldz + of + h] + b_f;
-      i = cap * tanhf(zi / cap);
-      const float u = cap * tanhf(zf / cap);
+      i = cap * tanhf(zi * inv_cap);
+      const float u = cap * tanhf(zf * inv_cap);
       f = fminf(u, 0.f) - log1pf(expf(-fabsf(u)));
     }
     float F = f, M = i;
@@ -44,26 +53,50 @@ exp_gates_kernel(const float* __restrict__ z, int ldz, int oi, int of, const flo
         F += Fb;
       }
     }
-    const float now = fmaxf(p + F, M);
-    const float up = __shfl_up(now, 1, 64), before = lane == 0 ? p : up;
-    if (live) {
+    float start = p;                                 // the maximum before this wavefront's tokens
+    if constexpr (W > 1) {
+      __syncthreads();                               // (the turn before has been read)
+      if (lane == 63) {
+        wf[wave] = F;
+        wi[wave] = M;
+      }
+      __syncthreads();
+#pragma unroll
+      for (int w = 0; w < W; ++w) {
+        if (w == wave) start = p;
+        p = fmaxf(p + wf[w], wi[w]);
+      }
+    } else {
+      p = fmaxf(p + __shfl(F, 63, 64), __shfl(M, 63, 64));
+    }
+    const float now = fmaxf(start + F, M);
+    const float up = __shfl_up(now, 1, 64), before = lane == 0 ? start : up;
+    if (in) {
       float* g = gates + (size_t)t * 3 * H + h;
-      g[0] = expf(f + before - now);
-      g[H] = expf(i - now);
+      const float keep = f + before - now, put = i - now;
+      g[0] = logs ? keep * MM_LOG2E : expf(keep);
+      g[H] = logs ? put * MM_LOG2E : expf(put);
       g[2 * H] = expf(-now);
     }
-    p = __shfl(now, t1 - tb < 64 ? t1 - tb - 1 : 63, 64);
   }
-  if (lane == 0) *own = p;
+  if (W == 1 ? lane == 0 : threadIdx.x == 0) *own = p;
 }
 
+// longest: the most tokens a sequence brings (how a launch is shaped, not what it computes)
 extern "C" int gs_exp_gates(const float* z, int ldz, int oi, int of, const float* bi, const float* bf, float cap, float* peak,
-                            const int* q_start, const int* slots, float* gates, int nseq, int H, hipStream_t stream) {
-  GS_REQUIRE(nseq >= 0 && H > 0 && H <= 4 * 65535, "exp_gates: bad sizes nseq=%d H=%d", nseq, H);
+                            const int* q_start, const int* slots, float* gates, int nseq, int H, int longest, int logs,
+                            hipStream_t stream) {
+  GS_REQUIRE(nseq >= 0 && H > 0 && H <= 65535, "exp_gates: bad sizes nseq=%d H=%d", nseq, H);
   GS_REQUIRE(oi >= 0 && of >= 0 && oi + H <= ldz && of + H <= ldz, "exp_gates: the gates' products lie outside the rows of %d", ldz);
   GS_REQUIRE(cap > 0.f, "exp_gates: the cap must be positive");
   if (nseq == 0) return 0;
-  exp_gates_kernel<<<dim3(nseq, gs_ceil_div(H, 4)), 256, 0, stream>>>(z, ldz, oi, of, bi, bf, cap, peak, q_start, slots, gates, H);
+#define GS_RUN(W, BLOCKS)                                                                                                   \
+  exp_gates_kernel<W><<<dim3(nseq, BLOCKS), W == 1 ? 256 : W * 64, 0, stream>>>(z, ldz, oi, of, bi, bf, cap, peak, q_start, \
+                                                                                slots, gates, H, logs)
+  if (longest <= 64) GS_RUN(1, gs_ceil_div(H, 4));
+  else if (longest <= 512) GS_RUN(4, H);
+  else GS_RUN(16, H);
+#undef GS_RUN
   GS_LAUNCH_CHECK("exp_gates");
   return 0;
 }
@@ -73,13 +106,14 @@ extern "C" int gs_exp_gates(const float* z, int ldz, int oi, int of, const float
 #define MM_KEEP 8
 template <typename TG, typename TO>
 __global__ void __launch_bounds__(256)
-memory_outnorm_kernel(const float* __restrict__ o, const float* __restrict__ gates, const TG* __restrict__ rows, int ldr,
+memory_outnorm_kernel(const float* __restrict__ o, int hs, const float* __restrict__ den, int ds,
+                      const float* __restrict__ gates, const TG* __restrict__ rows, int ldr,
                       int og, const float* __restrict__ w, float eps, TO* __restrict__ out, int H, int m) {
   const int t = blockIdx.x, lane = threadIdx.x & 63, nw = blockDim.x >> 6;
   for (int h = threadIdx.x >> 6; h < H; h += nw) {
-    const float* row = o + ((size_t)t * H + h) * (m + 1);
+    const float* row = o + ((size_t)t * H + h) * hs;
     const TG* gt = rows + (size_t)t * ldr + og + (size_t)h * m;
-    const float inv_den = 1.0f / (fmaxf(fabsf(row[m]), gates[(size_t)t * 3 * H + 2 * H + h]) + 1e-6f);
+    const float inv_den = 1.0f / (fmaxf(fabsf(den[((size_t)t * H + h) * ds]), gates[(size_t)t * 3 * H + 2 * H + h]) + 1e-6f);
     float keep[MM_KEEP], ss = 0.f;
 #pragma unroll
     for (int u = 0; u < MM_KEEP; ++u) {
@@ -104,19 +138,20 @@ memory_outnorm_kernel(const float* __restrict__ o, const float* __restrict__ gat
   }
 }
 
-extern "C" int gs_memory_outnorm(const float* o, const float* gates, const void* rows, int rows_dtype, int ldr, int og,
+extern "C" int gs_memory_outnorm(const float* o, int hs, const float* den, int ds, const float* gates, const void* rows, int rows_dtype, int ldr, int og,
                                  const float* w, float eps, void* out, int out_dtype, int T, int H, int m,
                                  hipStream_t stream) {
   GS_REQUIRE(T >= 0 && H > 0 && m > 0 && og >= 0 && og + H * m <= ldr, "memory_outnorm: bad sizes T=%d H=%d m=%d, or a gate outside the rows of %d", T, H, m, ldr);
+  GS_REQUIRE(hs >= m && ds > 0, "memory_outnorm: bad strides %d, %d", hs, ds);
   GS_REQUIRE(eps > 0.f, "memory_outnorm: eps must be positive");
   if (T == 0) return 0;
   const int threads = H >= 4 ? 256 : 64 * H;
   if (rows_dtype == GS_F32 && out_dtype == GS_F32)
-    memory_outnorm_kernel<float, float><<<T, threads, 0, stream>>>(o, gates, (const float*)rows, ldr, og, w, eps, (float*)out, H, m);
+    memory_outnorm_kernel<float, float><<<T, threads, 0, stream>>>(o, hs, den, ds, gates, (const float*)rows, ldr, og, w, eps, (float*)out, H, m);
   else if (rows_dtype == GS_BF16 && out_dtype == GS_BF16)
-    memory_outnorm_kernel<bf16, bf16><<<T, threads, 0, stream>>>(o, gates, (const bf16*)rows, ldr, og, w, eps, (bf16*)out, H, m);
+    memory_outnorm_kernel<bf16, bf16><<<T, threads, 0, stream>>>(o, hs, den, ds, gates, (const bf16*)rows, ldr, og, w, eps, (bf16*)out, H, m);
   else if (rows_dtype == GS_F32 && out_dtype == GS_BF16)
-    memory_outnorm_kernel<float, bf16><<<T, threads, 0, stream>>>(o, gates, (const float*)rows, ldr, og, w, eps, (bf16*)out, H, m);
+    memory_outnorm_kernel<float, bf16><<<T, threads, 0, stream>>>(o, hs, den, ds, gates, (const float*)rows, ldr, og, w, eps, (bf16*)out, H, m);
   else
     GS_REQUIRE(false, "memory_outnorm: unknown dtypes %d %d", rows_dtype, out_dtype);
   GS_LAUNCH_CHECK("memory_outnorm");

@@ -168,6 +168,66 @@ __global__ void qknorm_rope_kv_vec_kernel(T* __restrict__ qkv, const float* __re
   if (live && (is_q || write_kv)) store8f(o, v);
 }
 
+// Heads of other widths in whole pieces of eight, or rotated in part (rotary_dim a multiple of 16, half-split): P lanes per
+// (token, head), a power of two, of which the first d / 8 hold eight features each; a feature's partner lies rotary_dim / 16
+// lanes away, and lanes beyond the rotary part keep theirs.
+template <typename T, int P>
+__global__ void qknorm_rope_kv_part_kernel(T* __restrict__ qkv, const float* __restrict__ qw, const float* __restrict__ kw,
+                                           float eps, const float* __restrict__ cos_t, const float* __restrict__ sin_t,
+                                           int rotary_dim, const int* __restrict__ positions,
+                                           const int* __restrict__ seq_of_token, const int* __restrict__ block_table,
+                                           int max_blocks, int page_size, T* __restrict__ kcache, T* __restrict__ vcache,
+                                           int ntok, int nh, int nkv, int d, int write_kv, int ld) {
+  const int heads = nh + 2 * nkv;
+  const long unit = ((long)blockIdx.x * blockDim.x + threadIdx.x) / P;
+  const int sub = threadIdx.x % P;
+  const bool live = unit < (long)ntok * heads && sub * 8 < d;   // the others run along for the shuffles
+  const long un = unit < (long)ntok * heads ? unit : 0;
+  const int t = (int)(un / heads);
+  const int hh = (int)(un - (long)t * heads);
+  T* x = qkv + (size_t)t * ld + (size_t)hh * d + sub * 8;
+  const int pos = positions[t];
+  const bool is_q = hh < nh, is_k = !is_q && hh < nh + nkv;
+  T* o = x;
+  if (!is_q) {
+    const int kvh = is_k ? hh - nh : hh - nh - nkv;
+    const int page = block_table[(size_t)seq_of_token[t] * max_blocks + pos / page_size];
+    o = (is_k ? kcache : vcache) + (((size_t)page * nkv + kvh) * page_size + pos % page_size) * d + sub * 8;
+  }
+  float v[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+  if (live) load8f(x, v);
+  if (qw) {
+    float ss = 0.f;
+#pragma unroll
+    for (int k = 0; k < 8; ++k) ss += v[k] * v[k];
+#pragma unroll
+    for (int m = 1; m < P; m <<= 1) ss += __shfl_xor(ss, m, 64);
+    if (live && (is_q || is_k)) {
+      const float inv = norm_inverse(ss, (float)d, eps);
+      float w8[8];
+      load8f((is_q ? qw : kw) + sub * 8, w8);
+#pragma unroll
+      for (int k = 0; k < 8; ++k) v[k] = v[k] * inv * w8[k];
+    }
+  }
+  const int hp = rotary_dim >> 4, half = rotary_dim >> 1;       // lanes a half of the rotary part takes
+  const bool low = sub < hp, turned = sub < 2 * hp;
+  const int from = (threadIdx.x & 63) + (turned ? (low ? hp : -hp) : 0);
+  float other[8];
+#pragma unroll
+  for (int k = 0; k < 8; ++k) other[k] = __shfl(v[k], from, 64);
+  if (!live || (!is_q && !write_kv)) return;
+  if (turned && (is_q || is_k)) {
+    float c8[8], s8[8];
+    const int i0 = (low ? sub : sub - hp) * 8;
+    load8f(cos_t + (size_t)pos * half + i0, c8);
+    load8f(sin_t + (size_t)pos * half + i0, s8);
+#pragma unroll
+    for (int k = 0; k < 8; ++k) v[k] = low ? v[k] * c8[k] - other[k] * s8[k] : other[k] * s8[k] + v[k] * c8[k];
+  }
+  store8f(o, v);
+}
+
 extern "C" int gs_qknorm_rope_kv(void* qkv, int dtype, const float* qw, const float* kw, float eps,
                                  const float* cos_t, const float* sin_t, int rotary_dim, int interleaved,
                                  int max_position, const int* positions, const int* seq_of_token, const int* block_table,
@@ -216,6 +276,33 @@ extern "C" int gs_qknorm_rope_kv(void* qkv, int dtype, const float* qw, const fl
     if (dtype == GS_F32) { GS_VEC_T(float) } else { GS_VEC_T(bf16) }
 #undef GS_VEC_T
 #undef GS_VEC
+    GS_LAUNCH_CHECK("qknorm_rope_kv");
+    return 0;
+  }
+  const bool part = maps == 1 && !plain_norm && !v_first && !interleaved && vd == d && !vcos && d % 8 == 0 && d <= 256 &&
+                    rotary_dim % 16 == 0 && ld % 8 == 0 && (dtype == GS_F32 || dtype == GS_BF16) &&
+                    (((uintptr_t)qkv | (uintptr_t)kcache | (uintptr_t)vcache | (uintptr_t)cos_t | (uintptr_t)sin_t |
+                      (uintptr_t)qw | (uintptr_t)kw) & 15) == 0;
+  if (part) {
+    int P = 1;
+    while (P * 8 < d) P *= 2;
+    const int pblocks = gs_ceil_div(units * P, 256);
+#define GS_PART(T, PP)                                                                                                     \
+  qknorm_rope_kv_part_kernel<T, PP><<<pblocks, 256, 0, stream>>>((T*)qkv, qw, kw, eps, cos_t, sin_t, rotary_dim, positions, \
+                                                                 seq_of_token, block_table, max_blocks, page_size,         \
+                                                                 (T*)kcache, (T*)vcache, ntok, nh, nkv, d, write_kv, ld)
+#define GS_PART_T(T)                   \
+  switch (P) {                         \
+    case 1: GS_PART(T, 1); break;      \
+    case 2: GS_PART(T, 2); break;      \
+    case 4: GS_PART(T, 4); break;      \
+    case 8: GS_PART(T, 8); break;      \
+    case 16: GS_PART(T, 16); break;    \
+    default: GS_PART(T, 32); break;    \
+  }
+    if (dtype == GS_F32) { GS_PART_T(float) } else { GS_PART_T(bf16) }
+#undef GS_PART_T
+#undef GS_PART
     GS_LAUNCH_CHECK("qknorm_rope_kv");
     return 0;
   }

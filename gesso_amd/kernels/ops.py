@@ -1829,11 +1829,13 @@ def channel_decay(z, tau: float) -> torch.Tensor:
 
 # ---------------------------------------------------------------------- a matrix memory with exponential gates
 
-def exp_gates(z, oi: int, of: int, bias_i, bias_f, cap: float, peak, q_start, slots, nseq: int, H: int) -> torch.Tensor:
+def exp_gates(z, oi: int, of: int, bias_i, bias_f, cap: float, peak, q_start, slots, nseq: int, H: int, longest: int = 1,
+              logs: bool = False) -> torch.Tensor:
     """From float32 products ``z (T, ldz)`` (head ``h``'s input gate at ``[oi + h]``, its forget gate at ``[of + h]``):
     ``i = cap tanh((z + b) / cap)``, ``f = log sigmoid(cap tanh((z + b) / cap))``, the running maximum
     ``p_t = max(f + p_(t-1), i)`` from ``peak (slots, H)`` on, which it leaves there.  Returns float32 ``(T, 3 H)``:
-    ``exp(f + p_(t-1) - p_t)``, ``exp(i - p_t)``, ``exp(-p_t)``."""
+    ``exp(f + p_(t-1) - p_t)``, ``exp(i - p_t)`` (with ``logs`` the base-2 logarithms of these two), ``exp(-p_t)``.
+    ``longest``: the most tokens a sequence brings (how the launch is shaped)."""
     _dev(z, bias_i, bias_f, peak, q_start, slots)
     _need(z.dim() == 2 and z.dtype == torch.float32, "exp_gates: the products are float32 rows (T, ldz)")
     for b in (bias_i, bias_f):
@@ -1843,22 +1845,69 @@ def exp_gates(z, oi: int, of: int, bias_i, bias_f, cap: float, peak, q_start, sl
     _i32(slots, nseq, "slots")
     gates = torch.empty((z.shape[0], 3 * H), dtype=torch.float32, device=z.device)
     _check(lib().gs_exp_gates(_p(z), z.shape[1], oi, of, _p(bias_i), _p(bias_f), float(cap), _p(peak), _p(q_start), _p(slots),
-                              _p(gates), nseq, H, _stream()))
+                              _p(gates), nseq, H, int(longest), 1 if logs else 0, _stream()))
     return gates
 
 
-def memory_outnorm(o, gates, rows, og: int, weight, eps: float, H: int, m: int, out_dtype) -> torch.Tensor:
-    """``o (T, H (m + 1))`` float32, each head's ``m`` columns and ``n . q`` behind them, ``gates`` as :func:`exp_gates`
-    leaves them: ``u = o / (max(|n . q|, exp(-p)) + 1e-6)``, ``u / sqrt(mean(u^2) + eps) * weight * sigmoid(gate)`` per
+def memory_chunks_supports(x, n: int, m: int, oq: int, ok: int, ov: int) -> bool:
+    """Whether the matrix-core kernel of the matrix memory takes these rows (bfloat16, whole 16-byte pieces, keys up to 256
+    wide)."""
+    return (x.dtype == torch.bfloat16 and x.dim() == 2 and x.is_contiguous() and x.data_ptr() % 16 == 0
+            and bool(lib().gs_memory_chunks_supports(n, m, x.shape[1], oq, ok, ov)))
+
+
+def _memory_chunks(x, oq, ok, ov, H, n, m, logs, state, q_start, slots, nseq, q_scale, outputs: bool):
+    T, dev = x.shape[0], x.device
+    out = den = seg_d = None
+    if outputs:
+        out, den = torch.empty((T, H * m), dtype=torch.float32, device=dev), torch.empty((T, H), dtype=torch.float32, device=dev)
+    else:
+        seg_d = torch.empty(state.shape[:3], dtype=torch.float32, device=dev)
+    _check(lib().gs_memory_chunks(_p(x), x.shape[1], oq, ok, ov, float(q_scale), _p(logs), logs.shape[1], _p(state), _p(q_start),
+                                  _p(slots), _p(out), _p(den), _p(seg_d), nseq, H, n, m, _stream()))
+    return (out, den) if outputs else seg_d
+
+
+def memory_scan_chunks(x, oq: int, ok: int, ov: int, H: int, n: int, m: int, logs, state, q_start, slots, q_lens,
+                       q_scale: float = 1.0, segment: int = 0):
+    """The matrix memory's recurrence 32 tokens at a time on the matrix cores: :func:`gated_state_scan` with a decay a head,
+    write strengths, no delta rule and a column of ones (``state (slots, H, n, m + 1)``), the two gates given as base-2
+    logarithms in ``logs`` (:func:`exp_gates`).  Operands held in 32 bits enter as two bfloat16 terms.  ``segment`` > 0:
+    portions are cut into segments of that many tokens that run side by side (what each writes, starting from nothing; the
+    chain over a sequence's segments; the outputs from every segment's first state).  Returns float32 ``(T, H m)`` and the
+    last column's outputs ``(T, H)``."""
+    _dev(x, logs, state, q_start, slots)
+    nseq = len(q_lens)
+    _need(memory_chunks_supports(x, n, m, oq, ok, ov), "memory_scan_chunks: these rows are not taken (see memory_chunks_supports)")
+    _need(logs.dtype == torch.float32 and logs.dim() == 2 and logs.shape[0] == x.shape[0], "memory_scan_chunks: the gates are float32 rows")
+    _need(state.dtype == torch.float32 and state.dim() == 4 and state.shape[1:] == (H, n, m + 1),
+          "memory_scan_chunks: state must be float32 (slots, H, n, m + 1)")
+    _i32(q_start, nseq + 1, "q_start")
+    _i32(slots, nseq, "slots")
+    args = (x, oq, ok, ov, H, n, m, logs)
+    if segment <= 0:
+        return _memory_chunks(*args, state, q_start, slots, nseq, q_scale, True)
+    seg_start, seq_seg, ids, nseg = state_segment_tables(q_lens, segment, x.device)
+    B, first = torch.empty((2, nseg, H, n, m + 1), dtype=torch.float32, device=x.device)
+    D = _memory_chunks(*args, B, seg_start, ids, nseg, q_scale, False)
+    _check(lib().gs_gated_state_chain_diagonal(_p(D), _p(B), _p(first), _p(state), _p(seq_seg), _p(slots), nseq, H, n, m + 1, _stream()))
+    return _memory_chunks(*args, first, seg_start, ids, nseg, q_scale, True)
+
+
+def memory_outnorm(o, den, gates, rows, og: int, weight, eps: float, H: int, m: int, out_dtype) -> torch.Tensor:
+    """``o (T, H m)`` float32 and each head's ``n . q`` in ``den (T, H)``; or, with ``den = None``, ``o (T, H (m + 1))`` with
+    that number behind each head's columns.  With ``gates`` as :func:`exp_gates` leaves them: ``u = o / (max(|n . q|, exp(-p)) + 1e-6)``, ``u / sqrt(mean(u^2) + eps) * weight * sigmoid(gate)`` per
     head; the gate stands in ``rows`` from column ``og`` on.  Returns ``(T, H m)`` in ``out_dtype``."""
-    _dev(o, gates, rows, weight)
+    _dev(o, den, gates, rows, weight)
     T = o.shape[0]
-    _need(o.dtype == torch.float32 and o.shape == (T, H * (m + 1)), "memory_outnorm: o must be float32 (T, H (m + 1))")
+    hs = m if den is not None else m + 1
+    _need(o.dtype == torch.float32 and o.shape == (T, H * hs), "memory_outnorm: o must be float32 (T, H m), or (T, H (m + 1)) without den")
+    _need(den is None or (den.dtype == torch.float32 and den.shape == (T, H)), "memory_outnorm: den must be float32 (T, H)")
     _need(gates.dtype == torch.float32 and gates.shape == (T, 3 * H), "memory_outnorm: gates must be float32 (T, 3 H)")
     _need(rows.dim() == 2 and rows.shape[0] == T, "memory_outnorm: the gate's rows are (T, ld)")
     _need(weight.dtype == torch.float32 and weight.shape == (H * m,), "memory_outnorm: weight must be float32 (H m,)")
     out = torch.empty((T, H * m), dtype=out_dtype, device=o.device)
-    _check(lib().gs_memory_outnorm(_p(o), _p(gates), _p(rows), _dt(rows), rows.shape[1], og, _p(weight), float(eps), _p(out),
+    _check(lib().gs_memory_outnorm(_p(o), hs, _p(den) if den is not None else o.data_ptr() + 4 * m, 1 if den is not None else hs, _p(gates), _p(rows), _dt(rows), rows.shape[1], og, _p(weight), float(eps), _p(out),
                                    _dt(out), T, H, m, _stream()))
     return out
 

@@ -225,6 +225,8 @@ class GatedLinear(Part):
 class MatrixMemory(Part):
     graph_safe = True
     stage, out_stage = "memory_mixer", "memory_out"
+    RUNS_FROM = 8            # a step that brings a portion of at least this many tokens goes to the kernel on the matrix cores
+    SHORT_SEGMENT = 64
 
     def __init__(self, spec, rt):
         super().__init__(spec, rt)
@@ -263,13 +265,26 @@ class MatrixMemory(Part):
         x = rt.dense(x)
         with rt.stage("memory_in"):
             rows = rt.linear(x, self.w_in)                             # q | k | v | z (| spare columns)
+            runs = (rt.options.linear_attention == "auto" and not ctx.all_single and ctx.max_q_len >= self.RUNS_FROM
+                    and ops.memory_chunks_supports(rows, n, m, 0, H * n, 2 * H * n))
             gates = ops.exp_gates(rt.narrow_linear(x, self.w_gates), 0, H, self.b_i, self.b_f, s.gate_cap, cache.state["peak"],
-                                  ctx.q_start, ctx.slots, ctx.nseq, H)
+                                  ctx.q_start, ctx.slots, ctx.nseq, H, longest=ctx.max_q_len, logs=runs)
+        scale, den = float(n) ** -0.5, None
         with rt.stage("memory_state"):
-            o = _scan(ops, ctx, (rows, 0, H * n, 2 * H * n, H, H, n, m + 1, gates, 0, False), cache.state["state"],
-                      q_scale=float(n) ** -0.5, beta=gates, ob=H, delta=False, ones=True)
+            if runs:
+                # prompt portions 32 tokens at a time on the matrix cores; long ones in segments side by side, shorter
+                # segments where the longer ones would leave compute units without a block
+                seg = 0
+                if ctx.max_q_len >= 2 * self.SHORT_SEGMENT:
+                    blocks = sum(-(-L // SEGMENT) for L in ctx.q_lens) * H * -(-m // 128)
+                    seg = SEGMENT if blocks >= rt.compute_units else self.SHORT_SEGMENT
+                o, den = ops.memory_scan_chunks(rows, 0, H * n, 2 * H * n, H, n, m, gates, cache.state["state"], ctx.q_start,
+                                                ctx.slots, ctx.q_lens, q_scale=scale, segment=seg)
+            else:
+                o = _scan(ops, ctx, (rows, 0, H * n, 2 * H * n, H, H, n, m + 1, gates, 0, False), cache.state["state"],
+                          q_scale=scale, beta=gates, ob=H, delta=False, ones=True)
         with rt.stage("memory_norm"):
-            y = ops.memory_outnorm(o, gates, rows, 2 * H * n + H * m, self.norm_weight, s.eps, H, m, rt.dtype)
+            y = ops.memory_outnorm(o, den, gates, rows, 2 * H * n + H * m, self.norm_weight, s.eps, H, m, rt.dtype)
         return rt.linear(y, self.w_out, out_dtype=out_dtype)
 
 

@@ -47,7 +47,7 @@ class RuntimeOptions:
     the matrix cores once a step's (token, choice) pairs outnumber the experts twice over, ``"token"`` = token by token always.
     ``linear_attention``: linear attention through a fading state in bfloat16: ``"auto"`` = prompt portions 32 tokens at a
     time on the matrix cores (operands that the design holds in 32 bits as two bfloat16 terms), ``"token"`` = token by
-    token in float32 arithmetic always.
+    token in float32 arithmetic always.  The same for a matrix memory with exponential gates.
     ``tiled_rows``: rows handed from one fused kernel to the next product travel in the order the matrix cores
     take them (``ops.TiledRows``): a product then loads them a contiguous kilobyte at a time.
     ``tile_weights``: keep a tile-major copy of each bfloat16 weight for the streaming kernels.

@@ -44,7 +44,8 @@ class TokenSide(Part):
 
     def forward(self, x, ctx):
         rt, ops, s = self.rt, self.rt.ops, self.spec
-        z = rt.narrow_linear(x, self.w_gate)
+        # (a wide bottleneck is an ordinary product, its rows in the activation type)
+        z = rt.narrow_linear(x, self.w_gate) if self.width <= ops.NARROW_MAX_OUT else rt.linear(x, self.w_gate)
         g = ops.side_gate(z, self.table, ctx.token_ids, s.offset, s.dim, self.width, rt.dtype)
         return rt.linear(g, self.w_proj)
 
