@@ -150,6 +150,8 @@ extern "C" int gs_memory_outnorm(const float* o, int hs, const float* den, int d
     memory_outnorm_kernel<float, float><<<T, threads, 0, stream>>>(o, hs, den, ds, gates, (const float*)rows, ldr, og, w, eps, (float*)out, H, m);
   else if (rows_dtype == GS_BF16 && out_dtype == GS_BF16)
     memory_outnorm_kernel<bf16, bf16><<<T, threads, 0, stream>>>(o, hs, den, ds, gates, (const bf16*)rows, ldr, og, w, eps, (bf16*)out, H, m);
+  else if (rows_dtype == GS_BF16 && out_dtype == GS_F32)
+    memory_outnorm_kernel<bf16, float><<<T, threads, 0, stream>>>(o, hs, den, ds, gates, (const bf16*)rows, ldr, og, w, eps, (float*)out, H, m);
   else if (rows_dtype == GS_F32 && out_dtype == GS_BF16)
     memory_outnorm_kernel<float, bf16><<<T, threads, 0, stream>>>(o, hs, den, ds, gates, (const float*)rows, ldr, og, w, eps, (bf16*)out, H, m);
   else
