@@ -78,7 +78,7 @@ class BatchContext:
         for k, v in fields.items():
             setattr(self, k, v)
         self._storage = storage
-        self._tiles = None
+        self._tiles = {}           # tile lists by what they were cut for: mixers of several kinds each ask for their own
         self._segments = None
         # what one part of a step leaves for a later part of the same step (values that later layers blend with
         # theirs); empty at a step's start, gone at its end
@@ -98,7 +98,8 @@ class BatchContext:
     def query_tiles(self, rows: int = 16, skip: int = 0) -> torch.Tensor:
         """int32 ``(3, ntiles)``: sequence, first row, row count of each tile of at most ``rows`` consecutive
         queries of one sequence, for the sequences from ``skip`` on; made once per step, on first use."""
-        if self._tiles is None or self._tiles[0] != (rows, skip):
+        held = self._tiles.get((rows, skip))
+        if held is None:
             seq, row, cnt = [], [], []
             at = 0
             for i, n in enumerate(self.q_lens):
@@ -109,8 +110,8 @@ class BatchContext:
                         cnt.append(min(rows, n - a))
                 at += n
             t = torch.tensor([seq, row, cnt], dtype=torch.int32).pin_memory().to(self.token_ids.device, non_blocking=True)
-            self._tiles = ((rows, skip), t)
-        return self._tiles[1]
+            held = self._tiles[(rows, skip)] = t
+        return held
 
     def state_segments(self, seg_len: int):
         """The step's portions cut into segments of at most ``seg_len`` tokens, for recurrences that walk segments side by
@@ -134,10 +135,11 @@ class BatchContext:
     def query_subtiles(self, wq: int, skip: int = 0, paired: bool = True) -> torch.Tensor:
         """int32 ``(3, blocks * wq)`` on the device: :func:`subtile_lists` of this step's sequences from ``skip`` on."""
         key = ("sub", wq, skip, paired)
-        if self._tiles is None or self._tiles[0] != key:
+        held = self._tiles.get(key)
+        if held is None:
             t = torch.tensor(subtile_lists(self.q_lens, wq, skip, paired), dtype=torch.int32)
-            self._tiles = (key, t.pin_memory().to(self.token_ids.device, non_blocking=True))
-        return self._tiles[1]
+            held = self._tiles[key] = t.pin_memory().to(self.token_ids.device, non_blocking=True)
+        return held
 
 
 def subtile_lists(q_lens: Sequence[int], wq: int, skip: int = 0, paired: bool = True):

@@ -181,7 +181,7 @@ class RecordedStep:
         ctx = self.ctx
         ctx.q_lens = lens
         ctx.max_kv_len = int((held + lens_a).max())
-        ctx._tiles = None
+        ctx._tiles = {}
         if sum(len(e.want) for e in entries) > T:
             return None                                       # (rows wanted more than once: more than the buffer holds)
         self.turn = (self.turn + 1) % self.HOST_COPIES

@@ -1869,12 +1869,13 @@ def _memory_chunks(x, oq, ok, ov, H, n, m, logs, state, q_start, slots, nseq, q_
 
 
 def memory_scan_chunks(x, oq: int, ok: int, ov: int, H: int, n: int, m: int, logs, state, q_start, slots, q_lens,
-                       q_scale: float = 1.0, segment: int = 0):
+                       q_scale: float = 1.0, segment: int = 0, tables=None):
     """The matrix memory's recurrence 32 tokens at a time on the matrix cores: :func:`gated_state_scan` with a decay a head,
     write strengths, no delta rule and a column of ones (``state (slots, H, n, m + 1)``), the two gates given as base-2
     logarithms in ``logs`` (:func:`exp_gates`).  Operands held in 32 bits enter as two bfloat16 terms.  ``segment`` > 0:
     portions are cut into segments of that many tokens that run side by side (what each writes, starting from nothing; the
-    chain over a sequence's segments; the outputs from every segment's first state).  Returns float32 ``(T, H m)`` and the
+    chain over a sequence's segments; the outputs from every segment's first state); ``tables``: what
+    :func:`state_segment_tables` gives for them, where the caller has it.  Returns float32 ``(T, H m)`` and the
     last column's outputs ``(T, H)``."""
     _dev(x, logs, state, q_start, slots)
     nseq = len(q_lens)
@@ -1887,7 +1888,7 @@ def memory_scan_chunks(x, oq: int, ok: int, ov: int, H: int, n: int, m: int, log
     args = (x, oq, ok, ov, H, n, m, logs)
     if segment <= 0:
         return _memory_chunks(*args, state, q_start, slots, nseq, q_scale, True)
-    seg_start, seq_seg, ids, nseg = state_segment_tables(q_lens, segment, x.device)
+    seg_start, seq_seg, ids, nseg = tables or state_segment_tables(q_lens, segment, x.device)
     B, first = torch.empty((2, nseg, H, n, m + 1), dtype=torch.float32, device=x.device)
     D = _memory_chunks(*args, B, seg_start, ids, nseg, q_scale, False)
     _check(lib().gs_gated_state_chain_diagonal(_p(D), _p(B), _p(first), _p(state), _p(seq_seg), _p(slots), nseq, H, n, m + 1, _stream()))
@@ -1937,21 +1938,25 @@ def gemm_narrow(x, w: torch.Tensor, out_dtype=torch.float32) -> torch.Tensor:
 class SeamNorm:
     """A norm as :func:`norm_seam` takes it: ``("rms", w, eps)`` or ``("dyn_tanh", w, b, alpha)``."""
 
-    __slots__ = ("kind", "weight", "bias", "alpha", "eps")
+    __slots__ = ("kind", "weight", "bias", "alpha", "eps", "width", "passed")
     KINDS = {"rms": 1, "dyn_tanh": 2}
 
     def __init__(self, kind: str, weight, bias=None, alpha=None, eps: float = 0.0):
         self.kind, self.weight, self.bias, self.alpha, self.eps = self.KINDS[kind], weight, bias, alpha, float(eps)
+        self.width = None              # the width it has been checked for (once: a norm's tensors stay what they are)
 
     def check(self, H: int) -> None:
+        if self.width == H:
+            return
         ts = [self.weight] if self.kind == 1 else [self.weight, self.bias]
         _dev(*ts, self.alpha)
         _need(all(t is not None and t.dtype == torch.float32 and t.shape == (H,) for t in ts), "norm_seam: a norm's vectors are float32 (H,)")
         _need(self.kind == 1 or (self.alpha is not None and self.alpha.dtype == torch.float32 and self.alpha.numel() == 1),
               "norm_seam: alpha is one float32 number on the device")
+        self.width, self.passed = H, (self.kind, _p(self.weight), _p(self.bias), _p(self.alpha), self.eps)
 
     def args(self):
-        return self.kind, _p(self.weight), _p(self.bias), _p(self.alpha), self.eps
+        return self.passed
 
 
 _NO_SEAM_NORM = (0, None, None, None, 0.0)

@@ -274,12 +274,15 @@ class MatrixMemory(Part):
             if runs:
                 # prompt portions 32 tokens at a time on the matrix cores; long ones in segments side by side, shorter
                 # segments where the longer ones would leave compute units without a block
-                seg = 0
+                seg, tables = 0, None
                 if ctx.max_q_len >= 2 * self.SHORT_SEGMENT:
                     blocks = sum(-(-L // SEGMENT) for L in ctx.q_lens) * H * -(-m // 128)
                     seg = SEGMENT if blocks >= rt.compute_units else self.SHORT_SEGMENT
+                    tables = ctx.shared.get(("segments", seg))            # (one upload a step, whichever mixer asks first)
+                    if tables is None:
+                        tables = ctx.shared[("segments", seg)] = ops.state_segment_tables(ctx.q_lens, seg, rows.device)
                 o, den = ops.memory_scan_chunks(rows, 0, H * n, 2 * H * n, H, n, m, gates, cache.state["state"], ctx.q_start,
-                                                ctx.slots, ctx.q_lens, q_scale=scale, segment=seg)
+                                                ctx.slots, ctx.q_lens, q_scale=scale, segment=seg, tables=tables)
             else:
                 o = _scan(ops, ctx, (rows, 0, H * n, 2 * H * n, H, H, n, m + 1, gates, 0, False), cache.state["state"],
                           q_scale=scale, beta=gates, ob=H, delta=False, ones=True)
