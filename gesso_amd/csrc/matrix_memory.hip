@@ -12,6 +12,11 @@
 // few tokens: a wavefront per (sequence, head), four heads a block.  Longer portions: a block per (sequence, head), whose
 // wavefronts take 64 tokens each and hand their maps on through LDS.
 //
+// memory_step: one token a sequence.  A step then reads and writes every state once, and that stream is all the work: a block
+// owns 64 value columns of a (sequence, head), a wavefront a quarter of the rows, a lane a column, so that a row's columns
+// are read and written side by side; the wavefronts' shares of S^T q are added in order.  The state's last column (the sum of
+// the keys) goes along in the first column block, a thread a row.
+//
 // memory_outnorm: a head's m columns o and the number n . q (`den`), float32:
 //   u = o / (max(|n . q|, exp(-p)) + 1e-6);   out = u / sqrt(mean(u^2) + eps) * w * sigmoid(gate)      per head
 // Head h of token t has its columns at o[(t H + h) hs] and its number at den[(t H + h) ds].
@@ -98,6 +103,82 @@ extern "C" int gs_exp_gates(const float* z, int ldz, int oi, int of, const float
   else GS_RUN(16, H);
 #undef GS_RUN
   GS_LAUNCH_CHECK("exp_gates");
+  return 0;
+}
+
+#define MS_U 16           // rows a lane has in flight
+template <typename T>
+__global__ void __launch_bounds__(256)
+memory_step_kernel(const T* __restrict__ x, int ld, int oq, int ok, int ov, float q_scale, const float* __restrict__ gates,
+                   float* __restrict__ state, const int* __restrict__ slots, float* __restrict__ out,
+                   float* __restrict__ den, int H, int n, int m) {
+  extern __shared__ float ms_qk[];                    // q, then the weighted key, n each
+  __shared__ float part[4][64], red[17];
+  const int seq = blockIdx.x, h = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int j = blockIdx.z * 64 + lane, ms = m + 1;
+  const T* row = x + (size_t)seq * ld;
+  const float* g = gates + (size_t)seq * 3 * H + h;
+  const float keep = g[0], put = g[H];
+  float* S = state + ((size_t)slots[seq] * H + h) * n * ms;
+  float* q = ms_qk;
+  float* k = ms_qk + n;
+  for (int i = threadIdx.x; i < n; i += 256) {
+    q[i] = to_f32(row[oq + h * n + i]) * q_scale;
+    k[i] = to_f32(row[ok + h * n + i]) * put;
+  }
+  const bool col = j < m;
+  const float v = col ? to_f32(row[ov + h * m + j]) : 0.f;
+  __syncthreads();
+  const int per = (n + 3) / 4, i0 = wave * per, i1 = i0 + per < n ? i0 + per : n;
+  float acc = 0.f;
+  if (col) {
+    for (int ib = i0; ib < i1; ib += MS_U) {
+      float s[MS_U];
+#pragma unroll
+      for (int u = 0; u < MS_U; ++u) s[u] = S[(size_t)(ib + u < i1 ? ib + u : ib) * ms + j];
+#pragma unroll
+      for (int u = 0; u < MS_U; ++u) {
+        if (ib + u < i1) {
+          const float w = fmaf(k[ib + u], v, keep * s[u]);
+          S[(size_t)(ib + u) * ms + j] = w;
+          acc = fmaf(w, q[ib + u], acc);
+        }
+      }
+    }
+  }
+  part[wave][lane] = acc;
+  float d = 0.f;
+  if (blockIdx.z == 0)
+    for (int i = threadIdx.x; i < n; i += 256) {
+      const float w = fmaf(keep, S[(size_t)i * ms + m], k[i]);
+      S[(size_t)i * ms + m] = w;
+      d = fmaf(w, q[i], d);
+    }
+  __syncthreads();
+  if (wave == 0 && col) out[((size_t)seq * H + h) * m + j] = (part[0][lane] + part[1][lane]) + (part[2][lane] + part[3][lane]);
+  if (blockIdx.z == 0) {
+    d = block_sum(d, red);
+    if (threadIdx.x == 0) den[(size_t)seq * H + h] = d;
+  }
+}
+
+extern "C" int gs_memory_step(const void* x, int dtype, int ld, int oq, int ok, int ov, float q_scale, const float* gates,
+                              float* state, const int* slots, float* out, float* den, int nseq, int H, int n, int m,
+                              hipStream_t stream) {
+  GS_REQUIRE(nseq >= 0 && H > 0 && H <= 65535 && n > 0 && n <= 4096 && m > 0 && gs_ceil_div(m, 64) <= 65535,
+             "memory_step: bad sizes nseq=%d H=%d n=%d m=%d", nseq, H, n, m);
+  GS_REQUIRE(oq >= 0 && ok >= 0 && ov >= 0 && oq + H * n <= ld && ok + H * n <= ld && ov + H * m <= ld,
+             "memory_step: q, k or v lie outside the rows of %d", ld);
+  if (nseq == 0) return 0;
+  dim3 grid(nseq, H, gs_ceil_div(m, 64));
+  const size_t lds = 2 * (size_t)n * sizeof(float);
+  if (dtype == GS_F32)
+    memory_step_kernel<float><<<grid, 256, lds, stream>>>((const float*)x, ld, oq, ok, ov, q_scale, gates, state, slots, out, den, H, n, m);
+  else if (dtype == GS_BF16)
+    memory_step_kernel<bf16><<<grid, 256, lds, stream>>>((const bf16*)x, ld, oq, ok, ov, q_scale, gates, state, slots, out, den, H, n, m);
+  else
+    GS_REQUIRE(false, "memory_step: unknown dtype %d", dtype);
+  GS_LAUNCH_CHECK("memory_step");
   return 0;
 }
 

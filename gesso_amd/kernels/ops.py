@@ -1895,6 +1895,23 @@ def memory_scan_chunks(x, oq: int, ok: int, ov: int, H: int, n: int, m: int, log
     return _memory_chunks(*args, first, seg_start, ids, nseg, q_scale, True)
 
 
+def memory_step(x, oq: int, ok: int, ov: int, H: int, n: int, m: int, gates, state, slots, q_scale: float = 1.0):
+    """The matrix memory's recurrence for one token a sequence: row ``i`` of ``x`` is the next token of the sequence whose
+    memory lies in ``state[slots[i]]`` (``state (slots, H, n, m + 1)``), ``gates`` as :func:`exp_gates` leaves them.  Returns
+    float32 ``(nseq, H m)`` and the last column's outputs ``(nseq, H)``."""
+    _dev(x, gates, state, slots)
+    nseq = x.shape[0]
+    _need(gates.dtype == torch.float32 and gates.shape == (nseq, 3 * H), "memory_step: gates must be float32 (nseq, 3 H)")
+    _need(state.dtype == torch.float32 and state.dim() == 4 and state.shape[1:] == (H, n, m + 1),
+          "memory_step: state must be float32 (slots, H, n, m + 1)")
+    _i32(slots, nseq, "slots")
+    out = torch.empty((nseq, H * m), dtype=torch.float32, device=x.device)
+    den = torch.empty((nseq, H), dtype=torch.float32, device=x.device)
+    _check(lib().gs_memory_step(_p(x), _dt(x), x.shape[1], oq, ok, ov, float(q_scale), _p(gates), _p(state), _p(slots), _p(out), _p(den),
+                                nseq, H, n, m, _stream()))
+    return out, den
+
+
 def memory_outnorm(o, den, gates, rows, og: int, weight, eps: float, H: int, m: int, out_dtype) -> torch.Tensor:
     """``o (T, H m)`` float32 and each head's ``n . q`` in ``den (T, H)``; or, with ``den = None``, ``o (T, H (m + 1))`` with
     that number behind each head's columns.  With ``gates`` as :func:`exp_gates` leaves them: ``u = o / (max(|n . q|, exp(-p)) + 1e-6)``, ``u / sqrt(mean(u^2) + eps) * weight * sigmoid(gate)`` per

@@ -283,6 +283,8 @@ class MatrixMemory(Part):
                         tables = ctx.shared[("segments", seg)] = ops.state_segment_tables(ctx.q_lens, seg, rows.device)
                 o, den = ops.memory_scan_chunks(rows, 0, H * n, 2 * H * n, H, n, m, gates, cache.state["state"], ctx.q_start,
                                                 ctx.slots, ctx.q_lens, q_scale=scale, segment=seg, tables=tables)
+            elif ctx.all_single:
+                o, den = ops.memory_step(rows, 0, H * n, 2 * H * n, H, n, m, gates, cache.state["state"], ctx.slots, q_scale=scale)
             else:
                 o = _scan(ops, ctx, (rows, 0, H * n, 2 * H * n, H, H, n, m + 1, gates, 0, False), cache.state["state"],
                           q_scale=scale, beta=gates, ob=H, delta=False, ones=True)

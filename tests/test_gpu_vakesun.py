@@ -346,7 +346,8 @@ def test_gates_and_their_running_maximum_over_unequal_sequences_and_any_cut(ops,
 def memory_case(ops, dtype, H, n, m, lens, cuts, route, seed=0, segment=0, meet=None, slow=False):
     """A memory over sequences of ``lens`` tokens fed in the pieces ``cuts[s]``: gates, recurrence, and the divided, normed
     and gated outputs, states in shuffled slots.  ``route``: "scan" token by token (with ``segment`` in segments side by
-    side), "cores" 32 tokens at a time on the matrix cores.  ``meet``: ``(t, u)``: one key of token ``t`` is met by the query
+    side), "steps" the same with the kernel for single tokens where a step brings nothing else, "cores" 32 tokens at a time
+    on the matrix cores.  ``meet``: ``(t, u)``: one key of token ``t`` is met by the query
     of token ``u`` alone.  Returns the divided outputs' rows (with the gate at one half, no weight's effect) and the plain
     memory's, per sequence."""
     g = gen(seed)
@@ -386,7 +387,9 @@ def memory_case(ops, dtype, H, n, m, lens, cuts, route, seed=0, segment=0, meet=
         gates = ops.exp_gates(z, 0, H, zero, zero, 15.0, peak, starts, at, len(live), H, longest=max(sizes), logs=cores)
         offs = (junk, junk + H * n, junk + 2 * H * n)
         den = None
-        if cores:
+        if route == "steps" and all(k == 1 for k in sizes):
+            o, den = ops.memory_step(x, *offs, H, n, m, gates, state, at, q_scale=q_scale)
+        elif cores:
             o, den = ops.memory_scan_chunks(x, *offs, H, n, m, gates, state, starts, at, sizes, q_scale=q_scale, segment=segment)
         else:
             kw = dict(q_scale=q_scale, beta=gates, ob=H, delta=False, ones=True)
@@ -427,6 +430,20 @@ def test_the_memory_token_by_token_over_unequal_sequences_and_any_cut(ops, dtype
             assert near(got[s], want[s], 1e-4), (s, cuts[s][:2])
 
 
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H,n,m", [(4, 16, 24), (3, 8, 12), (2, 64, 128), (1, 128, 40), (5, 6, 14), (2, 13, 70), (1, 200, 33), (3, 32, 129), (2, 300, 8), (1, 1, 1)])
+def test_the_memory_one_token_a_sequence(ops, dtype, H, n, m):
+    """From nothing, and behind portions that the other kernels have walked."""
+    if n <= 256:
+        lens, cuts = [40, 23, 61], [[9] + [1] * 31, [23], [30] + [1] * 31]
+        got, want = memory_case(ops, dtype, H, n, m, lens, cuts, "steps", seed=n + m)
+        for s in range(len(lens)):
+            assert near(got[s], want[s], 1e-4), s
+    got, want = memory_case(ops, dtype, H, n, m, [30, 11], [[1] * 30, [1] * 11], "steps", seed=n + m + 1)
+    for s in range(2):
+        assert near(got[s], want[s], 1e-4), s
+
+
 @pytest.mark.parametrize("H,n,m,seg", [(2, 64, 128, 128), (4, 16, 24, 64), (1, 40, 10, 32)])
 def test_the_memory_in_segments_side_by_side(ops, H, n, m, seg):
     lens = [300, 1, 130, 64]
@@ -451,7 +468,7 @@ def test_the_memory_on_the_matrix_cores(ops, H, n, m, seg):
             assert near(got[s], want[s], 3e-3), (s, cuts[s][:2])
 
 
-@pytest.mark.parametrize("route,dtype,bound", [("scan", torch.float32, 2e-4), ("cores", torch.bfloat16, 3e-3)])
+@pytest.mark.parametrize("route,dtype,bound", [("scan", torch.float32, 2e-4), ("steps", torch.float32, 2e-4), ("cores", torch.bfloat16, 3e-3)])
 @pytest.mark.parametrize("cuts,seg", [([[420]], 0), ([[420]], 128), ([[40] + [1] * 380], 0), ([[200, 220]], 64)])
 def test_a_memory_keeps_what_it_was_given_hundreds_of_tokens_before(ops, route, dtype, bound, cuts, seg):
     """Nothing else has a share in the channel that the late query asks for: what it finds is the one value, 380 tokens old."""
